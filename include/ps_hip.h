@@ -312,6 +312,7 @@ enum ps_mixer_kind {
                          * a sink in the soft-max denominator, a temperature per head, norms over the whole q / k projections, partial rotary, a gate per head */
     PS_MIX_GLA    = 5, /* gated linear attention: S <- diag(alpha) S + k v^T, o = S^T q, a decay per key channel from a two-matrix projection */
     PS_MIX_MINGRU = 6, /* element-wise gated recurrence, its gates functions of the present input alone: S <- (1 - z) S + z c, output S * silu(g) */
+    PS_MIX_SSD    = 7, /* state-space recurrence with one decay per head (Mamba-2): S <- exp(-exp(a_log) dt) S + dt B x^T, y = S^T C + D x, gated and normed in parts */
 };
 enum ps_ff_kind {
     PS_FF_NONE = 0,
@@ -326,6 +327,8 @@ enum ps_layer_form {
     PS_LAYER_PARALLEL   = 1, /* h = norm1(x); x += res_scale (mixer(conv(h)) + ff(h2)): no norm behind the sublayers, only the mixer's input is filtered (canon1 NULL:
                               * not at all); h2 = h, or norm2(x) where norm2 is given (two weights over the same statistics) */
     PS_LAYER_PRENORM    = 2, /* x += mixer(norm1(x)), then x += ff(norm2(x)): the second norm reads what the mixer left; no input filter, nothing normed behind a sublayer */
+    PS_LAYER_POSTNORM   = 3, /* x += norm1b(mixer(x)), then x += norm2b(ff(x)): the sublayers read the residual stream itself, only their outputs are normed (a layer scale is folded into
+                              * the norm's weight); no input filter, norm1 / norm2 unused */
 };
 enum ps_rot_pairing { PS_ROT_HALVES = 0 /* (i, i + dims/2) */, PS_ROT_NEIGHBOURS = 1 /* (2i, 2i + 1) */ };
 
@@ -415,6 +418,22 @@ typedef struct ps_seq_layer_s {
      * only rows of the moe_keep best groups can be chosen.  moe_weight_output 1: a chosen expert's score multiplies its output (0: its input). */
     int32_t moe_identity, moe_softmax, moe_groups, moe_keep, moe_weight_output;
     const float *moe_correction;
+    float moe_scale;                    /* a chosen expert's weight is multiplied by this (0 is taken as 1; after moe_norm_top's division) */
+    /* ---- every mixer */
+    const float *out_bias;              /* [width] added by the output projection, or NULL */
+    /* ---- attention extras (PS_MIX_WINATTN), continued */
+    const float *dist_slope;            /* [heads] or NULL: dist_slope[h] * (i - j) is taken off the score of query position i and key position j, after scale and soft cap (no pooled blocks) */
+    int32_t keep_first;                 /* beside its window a position sees every j < keep_first up to itself (no pooled blocks); 0: none */
+    int32_t kv_from;                    /* 1 + the index of an earlier PS_MIX_WINATTN layer whose cached keys and values this layer reads (0: its own).  It then has queries only --
+                                         * in_cat = rows of q | gate, in_bias alike --, the same kv_heads, dim, vdim, and its own window, keep_first and everything else; the named layer
+                                         * has keys of its own, and there is no loop */
+    /* PS_MIX_LATENT reads rot_pairing too */
+    /* ---- PS_MIX_SSD; it reads heads, vdim (P), dim (the state size N), kv_heads (the groups that share B and C: head h reads group h / (heads / groups)), conv_taps, a_log, dt_bias
+     * [heads], onorm [heads * vdim], out.
+     *   in_cat = rows of z | x | B | C | dt  ([2*heads*vdim + 2*kv_heads*dim + heads, width]); conv [heads*vdim + 2*kv_heads*dim][conv_taps] and conv_bias (the same rows) over x | B | C, then silu;
+     *   dt = softplus(dt + dt_bias); the result times silu(z) is RMS-normed in norm_parts equal stretches, times onorm */
+    int32_t norm_parts;
+    const float *conv_bias, *skip;      /* skip: D [heads] */
 } ps_seq_layer;
 
 typedef struct {
@@ -433,6 +452,11 @@ typedef struct {
     int32_t max_context; /* most tokens a sequence may hold: sizes what grows with a sequence (the pooled blocks of PS_MIX_WINATTN, a window of everything); 0: 65536 */
     int32_t norm_groups; /* every RMS norm over the width is taken in this many equal consecutive parts, each with its own mean square (0 is taken as 1) */
     int32_t norm_center; /* 1: the norms over the width are layer norms -- the mean is taken off first and the variance is the mean of the squared deviations (PS_LAYER_PRENORM layers and the final norm) */
+    /* a second embedding table [bigram_buckets + 1, width], or NULL: row (previous token * bigram_mul_prev + token * bigram_mul_cur) mod bigram_buckets is added to the token's
+     * embedding, the last row for a sequence's first token (the previous token is part of a sequence's state) */
+    const ps_dense *bigram;
+    int64_t bigram_buckets, bigram_mul_prev, bigram_mul_cur;
+    float logit_softcap; /* logits <- logit_softcap * tanh(logits / logit_softcap), before logit_scale (0: none) */
 } ps_seq_desc;
 
 int ps_hip_seq_create(ps_hip_ctx *ctx, const ps_seq_desc *desc, ps_hip_seq **out);

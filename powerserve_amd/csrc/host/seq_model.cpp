@@ -442,8 +442,9 @@ void sink_attention_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploade
     L.sink = up.vec(std::vector<float>((size_t)L.heads, 0.f)); // exp(0) = 1 joins every head's denominator
     L.out = mat1(st, up, m + "o");
 }
-void shared_key_latent_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &m, const JsonValue &mc) {
+void shared_key_latent_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &m, const JsonValue &mc, int pairing = PS_ROT_HALVES) {
     L.kind = PS_MIX_LATENT;
+    L.rot_pairing = pairing;
     L.q_rank = 0; // the queries come straight from the input
     L.heads = (int32_t)mc.at("heads").num;
     L.dim = (int32_t)mc.at("dim").num;
@@ -503,6 +504,7 @@ void relu_feed_forward(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &
         L.top = (int32_t)r.at("top").num;
         L.moe_identity = (int32_t)num_or(r, "identity", 0);
         L.moe_softmax = 1;
+        L.moe_scale = (float)num_or(r, "scale", 1.0);
         L.moe_weight_output = 1;
         if (const JsonValue *gr = obj_or_null(r, "groups")) { L.moe_groups = (int32_t)num_or(*gr, "count", 0); L.moe_keep = (int32_t)num_or(*gr, "keep", 0); }
         const int rows = L.experts + L.moe_identity;
@@ -558,10 +560,130 @@ void pokatar(const JsonValue &cfg, const SafeTensorsFile &st, SeqUploader &up, s
         layers.push_back(L);
     }
 }
+// ---------------------------------------------------------------- Pupidra: post-norm layers, bigram embedding, state-space recurrence / windowed attention with first tokens / latent attention, scaled experts
+std::vector<float> stacked_bias(const SafeTensorsFile &st, const std::vector<std::string> &names, bool &any) { // zeros where a projection has none
+    std::vector<float> all;
+    any = false;
+    for (const auto &n : names) {
+        const int64_t r = rows_of(st, n);
+        if (st.contains(n + ".b")) { auto b = expect1(st, n + ".b", r); all.insert(all.end(), b.begin(), b.end()); any = true; }
+        else all.insert(all.end(), (size_t)r, 0.f);
+    }
+    return all;
+}
+// `layers`: all layers' configurations, of which this one is number `index` (kv_from names an earlier one)
+void kept_window_attention_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &m, const JsonValue &mc, const std::vector<JsonValue> &layers, size_t index) {
+    L.kind = PS_MIX_WINATTN;
+    L.heads = (int32_t)mc.at("heads").num;
+    L.dim = (int32_t)mc.at("dim").num;
+    L.kv_heads = (int32_t)num_or(mc, "kv_heads", L.heads);
+    L.vdim = (int32_t)num_or(mc, "vdim", L.dim);
+    if (L.kv_heads <= 0 || L.heads % L.kv_heads) POWERSERVE_ABORT(m + ": heads over key / value heads");
+    if (const JsonValue *mask = obj_or_null(mc, "mask")) { L.window = (int32_t)num_or(*mask, "size", 0); L.keep_first = (int32_t)num_or(*mask, "keep_first", 0); }
+    L.rot_pairing = PS_ROT_NEIGHBOURS;
+    L.rot_base = 10000.f;
+    L.scale = (float)num_or(mc, "scale", 1.0 / std::sqrt((double)L.dim));
+    L.head_norm = 1; // q and k divided by their root mean square per head, no weight
+    L.qnorm = up.vec(std::vector<float>((size_t)L.dim, 1.f));
+    std::vector<float> slope((size_t)L.heads); // what a token of distance costs a head's score
+    for (int h = 0; h < L.heads; h++) slope[(size_t)h] = (float)std::exp2(-8.0 * (h + 1.0) / L.heads);
+    L.dist_slope = up.vec(slope);
+    std::vector<std::string> names = {m + "q"};
+    check_rows(st, m + "q", (int64_t)L.heads * L.dim);
+    const int source = (int)num_or(mc, "kv_from", -1);
+    if (source < 0) {
+        L.knorm = up.vec(std::vector<float>((size_t)L.dim, 1.f));
+        check_rows(st, m + "k", (int64_t)L.kv_heads * L.dim);
+        check_rows(st, m + "v", (int64_t)L.kv_heads * L.vdim);
+        names.push_back(m + "k");
+        names.push_back(m + "v");
+    } else { // another layer's cached keys and values: queries only
+        if ((size_t)source >= index || layers[(size_t)source].at("type").str != "attention" || num_or(layers[(size_t)source].at("mixer"), "kv_from", -1) >= 0)
+            POWERSERVE_ABORT(m + ": kv_from names no earlier attention layer with keys of its own");
+        const JsonValue &of = layers[(size_t)source].at("mixer");
+        const double od = of.at("dim").num;
+        if (num_or(of, "kv_heads", of.at("heads").num) != L.kv_heads || od != L.dim || num_or(of, "vdim", od) != L.vdim) POWERSERVE_ABORT(m + ": kv_from: key / value sizes differ");
+        L.kv_from = source + 1;
+    }
+    L.in_cat = mat_rows(st, up, names);
+    bool any = false;
+    const auto bias = stacked_bias(st, names, any);
+    if (any) L.in_bias = up.vec(bias);
+    L.out = mat1(st, up, m + "o");
+    if (st.contains(m + "o.b")) L.out_bias = up.vec(expect1(st, m + "o.b", rows_of(st, m + "o")));
+}
+void state_space_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &m, const JsonValue &mc) {
+    L.kind = PS_MIX_SSD;
+    L.heads = (int32_t)mc.at("heads").num;
+    L.vdim = (int32_t)mc.at("vdim").num;
+    L.dim = (int32_t)mc.at("state").num;
+    L.kv_heads = (int32_t)num_or(mc, "groups", 1);
+    L.conv_taps = (int32_t)mc.at("conv").num;
+    L.norm_parts = (int32_t)num_or(mc, "norm_groups", 1);
+    const int64_t inner = (int64_t)L.heads * L.vdim, chan = inner + 2 * (int64_t)L.kv_heads * L.dim;
+    check_rows(st, m + "in", inner + chan + L.heads);
+    L.in_cat = mat1(st, up, m + "in");
+    L.out = mat1(st, up, m + "o");
+    L.conv = up.vec(expect(st, m + "conv", chan, L.conv_taps));
+    L.conv_bias = up.vec(st.contains(m + "conv.b") ? expect1(st, m + "conv.b", chan) : std::vector<float>((size_t)chan, 0.f));
+    L.a_log = up.vec(expect1(st, m + "A_log", L.heads));
+    L.dt_bias = up.vec(expect1(st, m + "dt_bias", L.heads));
+    L.skip = up.vec(expect1(st, m + "D", L.heads));
+    L.onorm = up.vec(expect1(st, m + "norm", inner));
+}
+void pupidra(const JsonValue &cfg, const SafeTensorsFile &st, SeqUploader &up, std::vector<ps_seq_layer> &layers, ps_seq_desc &d) {
+    d.width = (int32_t)cfg.at("width").num;
+    d.vocab = (int32_t)cfg.at("vocab").num;
+    d.canon_taps = 1;
+    d.norm_eps = (float)cfg.at("norm").at("eps").num;
+    d.norm_offset = 0.0f;
+    d.logit_scale = 1.0f;
+    d.logit_softcap = (float)num_or(cfg, "logit_softcap", 0.0);
+    d.loop_times = 1;
+    d.embed = mat1(st, up, "embed");
+    d.head = mat1(st, up, "head");
+    d.final_norm = up.vec(expect1(st, "final.norm", d.width));
+    const JsonValue *emb = obj_or_null(cfg, "embedding");
+    if (const JsonValue *big = emb ? obj_or_null(*emb, "bigram") : nullptr) {
+        d.bigram_buckets = (int64_t)big->at("buckets").num;
+        d.bigram_mul_prev = (int64_t)big->at("mul_prev").num;
+        d.bigram_mul_cur = (int64_t)big->at("mul_cur").num;
+        check_rows(st, "bigram", d.bigram_buckets + 1);
+        d.bigram = mat1(st, up, "bigram");
+    }
+    // RMS norm weight times layer scale: both multiply the normed output element by element
+    auto output_norm = [&](const std::string &p, const std::string &n) {
+        auto w = expect1(st, p + "norm" + n, d.width);
+        if (st.contains(p + "ls" + n)) {
+            const auto s = expect1(st, p + "ls" + n, d.width);
+            for (size_t i = 0; i < w.size(); i++) w[i] *= s[i];
+        }
+        return up.vec(w);
+    };
+    const auto &ls = cfg.at("layers").arr;
+    for (size_t i = 0; i < ls.size(); i++) {
+        const JsonValue &lc = ls[i], &mc = lc.at("mixer");
+        const std::string p = "l" + std::to_string(i) + ".", kind = lc.at("type").str;
+        ps_seq_layer L{};
+        L.form = PS_LAYER_POSTNORM;
+        L.mix_scale = 1.f;
+        L.norm1b = output_norm(p, "1");
+        if (kind == "mamba2") state_space_mixer(L, st, up, p + "mix.", mc);
+        else if (kind == "attention") kept_window_attention_mixer(L, st, up, p + "mix.", mc, ls, i);
+        else if (kind == "latent_attention") shared_key_latent_mixer(L, st, up, p + "mix.", mc, PS_ROT_NEIGHBOURS);
+        else POWERSERVE_ABORT("layer " + std::to_string(i) + ": mixer type " + kind + " is not known");
+        if (lc.contains("mlp") && lc.at("mlp").kind == JsonValue::OBJ) {
+            if (lc.at("mlp").at("kind").str != "moe") POWERSERVE_ABORT("layer " + std::to_string(i) + ": feed-forward kind " + lc.at("mlp").at("kind").str + " is not known");
+            L.norm2b = output_norm(p, "2");
+            relu_feed_forward(L, st, up, p + "mlp.", lc.at("mlp"), d.width);
+        }
+        layers.push_back(L);
+    }
+}
 } // namespace
 
 const std::map<std::string, SeqArchitecture> &seq_architectures() {
-    static const std::map<std::string, SeqArchitecture> reg = {{"Ranutar", ranutar}, {"Vobisun", vobisun}, {"Zusolix", zusolix}, {"Pokatar", pokatar}};
+    static const std::map<std::string, SeqArchitecture> reg = {{"Ranutar", ranutar}, {"Vobisun", vobisun}, {"Zusolix", zusolix}, {"Pokatar", pokatar}, {"Pupidra", pupidra}};
     return reg;
 }
 bool is_seq_model_dir(const std::string &dir) {

@@ -83,6 +83,8 @@ static __device__ __forceinline__ float dn_epi(const dn_args &g, float acc, long
         acc = tanhf(acc);
     } else if (g.act == PSD_ACT_RELU2) {
         acc = acc > 0.f ? acc * acc : 0.f;
+    } else if (g.act == PSD_ACT_SOFTCAP) {
+        acc = g.act_p * tanhf(acc / g.act_p);
     }
     return acc * g.alpha;
 }
@@ -579,16 +581,28 @@ void psk_dense_widen(hipStream_t st, const uint16_t *bf16, int64_t n, float *out
     hipLaunchKernelGGL(dense_widen_kernel, dim3((unsigned)blocks), dim3(256), 0, st, bf16, (long long)n, out);
 }
 
+static __device__ __forceinline__ float dn_table(const void *table, int is_bf16, long long i) {
+    return is_bf16 ? dn_bf2f(((const unsigned short *)table)[i]) : ((const float *)table)[i];
+}
+// bigram: a second table whose row depends on the previous and the present token (psk_embed)
 __global__ void dense_embed_kernel(const void *table, int is_bf16, long long K, const int32_t *tokens, const ps_seq_step *step, float scale, float *out,
-                                   long long ldo) {
+                                   long long ldo, const void *bigram, long long buckets, long long mul_prev, long long mul_cur) {
     const int t = blockIdx.x;
     const long long tok = (tokens ? tokens[t] : step->token0);
-    for (long long k = threadIdx.x; k < K; k += blockDim.x)
-        out[t * ldo + k] = (is_bf16 ? dn_bf2f(((const unsigned short *)table)[tok * K + k]) : ((const float *)table)[tok * K + k]) * scale;
+    long long row = 0;
+    if (bigram) {
+        const long long prev = t ? tokens[t - 1] : step->prev;
+        row = step->pos0 + t == 0 ? buckets : (prev * mul_prev + tok * mul_cur) % buckets;
+    }
+    for (long long k = threadIdx.x; k < K; k += blockDim.x) {
+        const float v = dn_table(table, is_bf16, tok * K + k) * scale;
+        out[t * ldo + k] = bigram ? v + dn_table(bigram, is_bf16, row * K + k) : v;
+    }
 }
-void psk_embed(hipStream_t st, const ps_dense *table, const int32_t *tokens, const ps_seq_step *step, int T, float scale, float *out, int64_t ldo) {
+void psk_embed(hipStream_t st, const ps_dense *table, const int32_t *tokens, const ps_seq_step *step, int T, float scale, float *out, int64_t ldo, const ps_dense *bigram,
+               int64_t buckets, int64_t mul_prev, int64_t mul_cur) {
     hipLaunchKernelGGL(dense_embed_kernel, dim3(T), dim3(256), 0, st, table->data, table->dtype == PS_BF16 ? 1 : 0, (long long)table->K, tokens, step, scale, out,
-                       (long long)ldo);
+                       (long long)ldo, bigram ? bigram->data : nullptr, (long long)buckets, (long long)mul_prev, (long long)mul_cur);
 }
 
 __global__ __launch_bounds__(256) void dense_argmax_kernel(const float *x, long long n, int32_t *out) {

@@ -21,9 +21,15 @@ static __device__ __forceinline__ float la_wave_max(float v) {
     return v;
 }
 
+// the two numbers of rotated pair i of a part whose first 2 half numbers turn
+static __device__ __forceinline__ void la_pair(int i, int half, int pairing, int &a, int &b) {
+    if (pairing == PS_ROT_NEIGHBOURS) { a = 2 * i; b = a + 1; }
+    else { a = i; b = i + half; }
+}
+
 __global__ __launch_bounds__(256) void latent_prep_kernel(const ps_seq_step *step, long long ring_off, int cap, const float *y, long long ldy, const float *qnorm,
                                                           const float *kvnorm, float eps, int q_rank, int kv_rank, int rot_dim, int rot_dims, const float *freq, float *cq,
-                                                          long long ldcq, float rot_mag) {
+                                                          long long ldcq, float rot_mag, int pairing) {
     __shared__ float red[8];
     const int t = blockIdx.x, tid = threadIdx.x;
     const long long pos = step->pos0 + t;
@@ -40,26 +46,28 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const ps_seq_step *ste
     const float ib = 1.f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)kv_rank + eps);
     for (int i = tid; i < q_rank; i += 256) cq[(long long)t * ldcq + i] = yt[i] * ia * qnorm[i];
     for (int i = tid; i < kv_rank; i += 256) ring[i] = ckv[i] * ib * kvnorm[i];
-    const int half = rot_dims / 2; // the first rot_dims of the part are rotated, pairs (i, i + rot_dims / 2); the rest passes unchanged
+    const int half = rot_dims / 2; // the first rot_dims of the part are rotated; the rest passes unchanged
     for (int i = tid; i < half; i += 256) {
         const float ang = (float)pos * freq[i], c = cosf(ang) * rot_mag, s = sinf(ang) * rot_mag;
-        const float u = kr[i], v = kr[i + half];
-        ring[kv_rank + i] = u * c - v * s;
-        ring[kv_rank + half + i] = v * c + u * s;
+        int pa, pb;
+        la_pair(i, half, pairing, pa, pb);
+        const float u = kr[pa], v = kr[pb];
+        ring[kv_rank + pa] = u * c - v * s;
+        ring[kv_rank + pb] = v * c + u * s;
     }
     for (int i = 2 * half + tid; i < rot_dim; i += 256) ring[kv_rank + i] = kr[i];
 }
 void psk_latent_prep(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, const float *y, int64_t ldy, const float *qnorm, const float *kvnorm,
-                     float eps, int q_rank, int kv_rank, int rot_dim, int rot_dims, const float *freq, int T, float *cq, int64_t ldcq, float rot_mag) {
+                     float eps, int q_rank, int kv_rank, int rot_dim, int rot_dims, const float *freq, int T, float *cq, int64_t ldcq, float rot_mag, int pairing) {
     hipLaunchKernelGGL(latent_prep_kernel, dim3(T), dim3(256), 0, st, step, (long long)ring_off, cap, y, (long long)ldy, qnorm, kvnorm, eps, q_rank, kv_rank, rot_dim,
-                       rot_dims, freq, cq, (long long)ldcq, rot_mag);
+                       rot_dims, freq, cq, (long long)ldcq, rot_mag, pairing);
 }
 
 // dynamic LDS: qs [d + dr], ps [64]
 #define LA_NV 4 // value columns per lane: dv <= 256
 __global__ __launch_bounds__(64) void latent_attn_kernel(const ps_seq_step *step, long long ring_off, int cap, const float *q, long long ldq, const float *kv,
                                                          long long ldkv, const float *freq, int H, int d, int dr, int rot_dims, int dv, int kv_rank, int window,
-                                                         float scale, float *o, long long ldo, float rot_mag, const float *gate, long long ldg) {
+                                                         float scale, float *o, long long ldo, float rot_mag, const float *gate, long long ldg, int pairing) {
     extern __shared__ float lds[];
     float *qs = lds, *ps = lds + d + dr;
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -72,9 +80,11 @@ __global__ __launch_bounds__(64) void latent_attn_kernel(const ps_seq_step *step
     for (int i = 2 * half + lane; i < dr; i += 64) qs[d + i] = qt[d + i];
     for (int i = lane; i < half; i += 64) {
         const float ang = (float)p * freq[i], c = cosf(ang) * rot_mag, s = sinf(ang) * rot_mag;
-        const float u = qt[d + i], v = qt[d + half + i];
-        qs[d + i] = u * c - v * s;
-        qs[d + half + i] = v * c + u * s;
+        int pa, pb;
+        la_pair(i, half, pairing, pa, pb);
+        const float u = qt[d + pa], v = qt[d + pb];
+        qs[d + pa] = u * c - v * s;
+        qs[d + pb] = v * c + u * s;
     }
     __syncthreads();
     const float *ring = step->state + ring_off;
@@ -118,9 +128,9 @@ __global__ __launch_bounds__(64) void latent_attn_kernel(const ps_seq_step *step
 }
 void psk_latent_attn(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, const float *q, int64_t ldq, const float *kv, int64_t ldkv,
                      const float *freq, int H, int d, int dr, int rot_dims, int dv, int kv_rank, int window, float scale, int T, float *o, int64_t ldo, float rot_mag,
-                     const float *gate, int64_t ldg) {
+                     const float *gate, int64_t ldg, int pairing) {
     hipLaunchKernelGGL(latent_attn_kernel, dim3(T, H), dim3(64), (size_t)(d + dr + 64) * 4, st, step, (long long)ring_off, cap, q, (long long)ldq, kv, (long long)ldkv,
-                       freq, H, d, dr, rot_dims, dv, kv_rank, window, scale, o, (long long)ldo, rot_mag, gate, (long long)ldg);
+                       freq, H, d, dr, rot_dims, dv, kv_rank, window, scale, o, (long long)ldo, rot_mag, gate, (long long)ldg, pairing);
 }
 
 // ---------------------------------------------------------------------------------------------------- matrix-core form
@@ -139,7 +149,7 @@ void psk_latent_attn(hipStream_t st, const ps_seq_step *step, int64_t ring_off, 
 template <int NJ>
 __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const ps_seq_step *step, long long ring_off, int cap, const float *q, long long ldq, const float *kv,
                                                                long long ldkv, const float *freq, int H, int d, int dr, int rot_dims, int dv, int kv_rank, int window,
-                                                               float scale, int T, float *o, long long ldo, float rot_mag, const float *gate, long long ldg) {
+                                                               float scale, int T, float *o, long long ldo, float rot_mag, const float *gate, long long ldg, int pairing) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lr = lane & 15, lq = lane >> 4, h = blockIdx.y;
     const int qld = d + dr + 4;
@@ -159,9 +169,11 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const ps_seq_step
         for (int c = 2 * half + lane; c < dr; c += 64) qr[d + c] = in ? qt[d + c] : 0.f;
         for (int i = lane; i < half; i += 64) {
             const float ang = (float)(pos0 + t) * freq[i], cs = cosf(ang) * rot_mag, sn = sinf(ang) * rot_mag;
-            const float u = in ? qt[d + i] : 0.f, v = in ? qt[d + half + i] : 0.f;
-            qr[d + i] = u * cs - v * sn;
-            qr[d + half + i] = v * cs + u * sn;
+            int pa, pb;
+            la_pair(i, half, pairing, pa, pb);
+            const float u = in ? qt[d + pa] : 0.f, v = in ? qt[d + pb] : 0.f;
+            qr[d + pa] = u * cs - v * sn;
+            qr[d + pb] = v * cs + u * sn;
         }
     }
     __builtin_amdgcn_wave_barrier();
@@ -199,12 +211,12 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const ps_seq_step
 bool psk_latent_attn_mfma_ok(int d, int dr, int dv) { return d % 16 == 0 && dr % 16 == 0 && dv % 4 == 0 && dv <= 128 && (size_t)4 * (16 * (d + dr + 4) + 16 * 17) * 4 <= 160 * 1024; }
 void psk_latent_attn_mfma(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, const float *q, int64_t ldq, const float *kv, int64_t ldkv,
                           const float *freq, int H, int d, int dr, int rot_dims, int dv, int kv_rank, int window, float scale, int T, float *o, int64_t ldo, float rot_mag,
-                          const float *gate, int64_t ldg) {
+                          const float *gate, int64_t ldg, int pairing) {
     const size_t lds = (size_t)4 * (16 * (d + dr + 4) + 16 * 17) * 4;
     static unsigned long long mask = 0;
     if (ps_first_on_device(&mask)) (void)hipFuncSetAttribute((const void *)latent_attn_mfma_kernel<8>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     hipLaunchKernelGGL(latent_attn_mfma_kernel<8>, dim3((T + 63) / 64, H), dim3(256), lds, st, step, (long long)ring_off, cap, q, (long long)ldq, kv, (long long)ldkv, freq,
-                       H, d, dr, rot_dims, dv, kv_rank, window, scale, T, o, (long long)ldo, rot_mag, gate, (long long)ldg);
+                       H, d, dr, rot_dims, dv, kv_rank, window, scale, T, o, (long long)ldo, rot_mag, gate, (long long)ldg, pairing);
 }
 
 // ---------------------------------------------------------------------------------------------------- single token, absorbed
@@ -249,7 +261,7 @@ __global__ __launch_bounds__(256) void latent_unfold_v_kernel(const float *ol, c
 // per (key tile, head) R unnormalised outputs, then m and l.  dynamic LDS: 16 x qld + 4 x 16 x 17
 template <int NJ>
 __global__ __launch_bounds__(256) void latent_absorbed_kernel(const ps_seq_step *step, long long ring_off, int cap, const float *qa, const float *q, int qstride, int d,
-                                                              int dr, int rot_dims, const float *freq, int H, int R, int window, float scale, float *part, float rot_mag) {
+                                                              int dr, int rot_dims, const float *freq, int H, int R, int window, float scale, float *part, float rot_mag, int pairing) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lr = lane & 15, lq = lane >> 4, h0 = blockIdx.y * 16;
     const int qld = R + dr + 4;
@@ -266,12 +278,14 @@ __global__ __launch_bounds__(256) void latent_absorbed_kernel(const ps_seq_step 
     }
     for (int i = lane; i < half; i += 64) {
         const float ang = (float)p * freq[i], cs = cosf(ang) * rot_mag, sn = sinf(ang) * rot_mag;
+        int pa, pb;
+        la_pair(i, half, pairing, pa, pb);
         for (int r = wave; r < 16; r += 4) {
             const int h = h0 + r;
             const float *qt = q + (long long)(h < H ? h : 0) * qstride + d;
-            const float u = h < H ? qt[i] : 0.f, v = h < H ? qt[half + i] : 0.f;
-            qs[r * qld + R + i] = u * cs - v * sn;
-            qs[r * qld + R + half + i] = v * cs + u * sn;
+            const float u = h < H ? qt[pa] : 0.f, v = h < H ? qt[pb] : 0.f;
+            qs[r * qld + R + pa] = u * cs - v * sn;
+            qs[r * qld + R + pb] = v * cs + u * sn;
         }
     }
     __syncthreads();
@@ -338,7 +352,7 @@ bool psk_latent_absorbed_ok(int d, int dr, int dv, int R) { return R % 16 == 0 &
 size_t psk_latent_absorbed_scratch(int H, int R, int window) { return ((size_t)((window + 15) / 16 + 4) * H * (R + 4) + (size_t)2 * H * R) * 4; }
 // q [H][d + dr] (row stride qstride) -> o [H * dv]; ukv: rows uk | uv of the expansion matrix [H d + H dv][R]; scratch from psk_latent_absorbed_scratch
 void psk_latent_absorbed(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, const float *q, int qstride, const ps_dense *ukv, const float *freq,
-                         int H, int d, int dr, int rot_dims, int dv, int R, int window, float scale, float *scratch, float *o, float rot_mag, const float *gate) {
+                         int H, int d, int dr, int rot_dims, int dv, int R, int window, float scale, float *scratch, float *o, float rot_mag, const float *gate, int pairing) {
     const int max_tiles = (window + 15) / 16 + 1; // (a window that does not start on a tile's edge touches one tile more)
     float *qa = scratch, *ol = qa + (size_t)H * R, *part = ol + (size_t)H * R;
     const bool bf = ukv->dtype == PS_BF16;
@@ -349,11 +363,11 @@ void psk_latent_absorbed(hipStream_t st, const ps_seq_step *step, int64_t ring_o
     if (R <= 128) {
         static unsigned long long mask = 0;
         if (ps_first_on_device(&mask)) (void)hipFuncSetAttribute((const void *)latent_absorbed_kernel<8>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-        hipLaunchKernelGGL(latent_absorbed_kernel<8>, grid, dim3(256), lds, st, step, (long long)ring_off, cap, qa, q, qstride, d, dr, rot_dims, freq, H, R, window, scale, part, rot_mag);
+        hipLaunchKernelGGL(latent_absorbed_kernel<8>, grid, dim3(256), lds, st, step, (long long)ring_off, cap, qa, q, qstride, d, dr, rot_dims, freq, H, R, window, scale, part, rot_mag, pairing);
     } else {
         static unsigned long long mask = 0;
         if (ps_first_on_device(&mask)) (void)hipFuncSetAttribute((const void *)latent_absorbed_kernel<32>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-        hipLaunchKernelGGL(latent_absorbed_kernel<32>, grid, dim3(256), lds, st, step, (long long)ring_off, cap, qa, q, qstride, d, dr, rot_dims, freq, H, R, window, scale, part, rot_mag);
+        hipLaunchKernelGGL(latent_absorbed_kernel<32>, grid, dim3(256), lds, st, step, (long long)ring_off, cap, qa, q, qstride, d, dr, rot_dims, freq, H, R, window, scale, part, rot_mag, pairing);
     }
     hipLaunchKernelGGL(latent_combine_kernel, dim3(H), dim3(256), (size_t)grid.x * 4 * 4, st, step, part, H, R, window, (int)grid.x * 4, ol);
     const int rows = H * dv;

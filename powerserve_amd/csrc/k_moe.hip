@@ -1,7 +1,7 @@
 // Mixture-of-experts routing for the layer-list models (PS_FF_MOE_SWIGLU, PS_FF_MOE_RELU2).  The experts' matrix products are grouped launches of the dense kernels
 // (k_dense.hip); here is what decides who goes where, all fp32:
-//   moe_route_kernel    a block per token: router logits, sigmoid or soft-max scores, a correction and a group limit on the choice, the `top` largest,
-//                       the shared expert's gate
+//   moe_route_kernel    a block per token: router logits, sigmoid or soft-max scores, a correction and a group limit on the choice, the `top` largest
+//                       (their scores times a constant), the shared expert's gate
 //   moe_plan_kernel     the token-expert slots sorted by expert (counts, offsets, list) for the tiled products
 //   moe_combine_kernel  a token's `top` per-slot results summed into the residual stream; an identity expert's share is its weight times the input
 #include "ps_seq.h"
@@ -21,8 +21,8 @@ typedef float moe_f4 __attribute__((ext_vector_type(4)));
 // groups that stay in the race, and `top` rounds of (largest choice score, lowest index); the weights are the SCORES of the chosen.
 // dynamic LDS: [rows + 1] scores, [rows] choice scores, [groups] group scores.
 __global__ __launch_bounds__(256) void moe_route_kernel(const float *h, long long ldh, const float *router, const float *shared_gate, int experts, int top, int norm_top,
-                                                        long long K, int softmax, const float *correction, int n_groups, int keep, int32_t *sel, float *wgt,
-                                                        float *sgate) {
+                                                        long long K, int softmax, const float *correction, int n_groups, int keep, float scale, int32_t *sel,
+                                                        float *wgt, float *sgate) {
     extern __shared__ float sc[];
     float *ch = sc + experts + 1, *gs = ch + experts;
     const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -111,17 +111,18 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float *h, long lon
         agree(best, at);
         const bool any = at != 0x7fffffff; // (nothing left in the race: the slot goes to row 0 with weight 0)
         const float w = any ? sc[at] : 0.f;
-        if (lane == 0) { sel[(long long)t * top + i] = any ? at : 0; wgt[(long long)t * top + i] = w; if (any) ch[at] = -INFINITY; }
+        if (lane == 0) { sel[(long long)t * top + i] = any ? at : 0; wgt[(long long)t * top + i] = norm_top ? w : w * scale; if (any) ch[at] = -INFINITY; }
         total += w;
         __builtin_amdgcn_wave_barrier();
         __threadfence_block();
     }
-    if (norm_top && lane < top) wgt[(long long)t * top + lane] /= total;
+    if (norm_top)
+        for (int i = lane; i < top; i += 64) wgt[(long long)t * top + i] = wgt[(long long)t * top + i] / total * scale;
 }
 void psk_moe_route(hipStream_t st, const float *h, int64_t ldh, const float *router, const float *shared_gate, int experts, int top, int norm_top, int64_t K, int T,
-                   int32_t *sel, float *wgt, float *sgate, int softmax, const float *correction, int n_groups, int keep) {
+                   int32_t *sel, float *wgt, float *sgate, int softmax, const float *correction, int n_groups, int keep, float scale) {
     hipLaunchKernelGGL(moe_route_kernel, dim3(T), dim3(256), (size_t)(2 * experts + 1 + (n_groups > 0 ? n_groups : 0)) * 4, st, h, (long long)ldh, router, shared_gate,
-                       experts, top, norm_top, (long long)K, softmax, correction, n_groups, keep, sel, wgt, sgate);
+                       experts, top, norm_top, (long long)K, softmax, correction, n_groups, keep, scale, sel, wgt, sgate);
 }
 
 // one block; dynamic LDS: 2 x experts ints.  Counts, offsets, then every slot takes the next free place of its expert.  Which place a slot gets is up to the
@@ -147,9 +148,9 @@ void psk_moe_plan(hipStream_t st, const int32_t *sel, int S, int experts, int32_
 }
 
 // x[t] += alpha * sum_k (slot t top + k: its product's result y[slot], or -- a slot whose choice is an identity expert, sel >= n_real -- wgt[slot] * h[t]);
-// y NULL: the products have been added already and only the identity slots are left.
+// y NULL: the products have been added already and only the identity slots are left.  store: x[t] = instead of +=.
 __global__ void moe_combine_kernel(float *x, const float *y, int top, float alpha, long long n, const int32_t *sel, const float *wgt, int n_real, const float *h,
-                                   long long ldh) {
+                                   long long ldh, int store) {
     const long long t = blockIdx.x;
     for (long long i = threadIdx.x; i < n; i += blockDim.x) {
         float a = 0.f;
@@ -158,10 +159,10 @@ __global__ void moe_combine_kernel(float *x, const float *y, int top, float alph
             if (sel && sel[s] >= n_real) a = fmaf(wgt[s], h[t * ldh + i], a);
             else if (y) a += y[s * n + i];
         }
-        x[t * n + i] += alpha * a;
+        x[t * n + i] = store ? alpha * a : x[t * n + i] + alpha * a;
     }
 }
 void psk_moe_combine(hipStream_t st, float *x, const float *y, int top, float alpha, int64_t n, int T, const int32_t *sel, const float *wgt, int n_real, const float *h,
-                     int64_t ldh) {
-    hipLaunchKernelGGL(moe_combine_kernel, dim3(T), dim3(256), 0, st, x, y, top, alpha, (long long)n, sel, wgt, n_real, h, (long long)ldh);
+                     int64_t ldh, int store) {
+    hipLaunchKernelGGL(moe_combine_kernel, dim3(T), dim3(256), 0, st, x, y, top, alpha, (long long)n, sel, wgt, n_real, h, (long long)ldh, store);
 }

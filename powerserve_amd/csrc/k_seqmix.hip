@@ -1,5 +1,5 @@
 // Mechanisms of the layer-list models that are not matrix products: RMS norms (with the residual add), causal convolutions over time
-// with a per-sequence tail, and the two recurrent scans (wkv, gated delta rule).  Everything here is fp32.
+// with a per-sequence tail, and the recurrent scans (wkv, gated linear attention, gated delta rule, state space, element-wise).  Everything here is fp32.
 //
 // The scans: a head's state S [d][dv] is split by COLUMN over threads -- every column j evolves on its own in both recurrences
 // (S_ij <- decay S_ij + k_i x_j needs only column j) -- and each column over R lanes of 16 rows each, so a step is 16 fused
@@ -122,13 +122,13 @@ static __device__ __forceinline__ void sq_conv_tail(float *tail, const float *in
     }
 }
 __global__ __launch_bounds__(256) void sq_conv_kernel(const ps_seq_step *step, long long tail_off, const float *in, long long ldi, const float *w, int taps, int mode,
-                                                      long long C, int T, float *out, long long ldo) {
+                                                      long long C, int T, float *out, long long ldo, const float *bias) {
     const long long c = (long long)blockIdx.x * 256 + threadIdx.x;
     if (c >= C) return;
     float *tail = step->state + tail_off;
     const int tb = blockIdx.y * SQ_CONV_CHUNK, te = min(T, tb + SQ_CONV_CHUNK);
     for (int t = tb; t < te; t++) {
-        float s = 0.f;
+        float s = bias ? bias[c] : 0.f;
         for (int j = 0; j < taps; j++) {
             const int r = t - taps + 1 + j;
             const float v = r >= 0 ? in[(long long)r * ldi + c] : tail[(long long)(taps - 1 + r) * C + c];
@@ -143,9 +143,9 @@ __global__ __launch_bounds__(256) void sq_conv_tail_kernel(const ps_seq_step *st
     if (c < C) sq_conv_tail(step->state + tail_off, in, ldi, taps, C, T, c);
 }
 void psk_causal_conv(hipStream_t st, const ps_seq_step *step, int64_t tail_off, const float *in, int64_t ldi, const float *w, int taps, int mode, int64_t C, int T,
-                     float *out, int64_t ldo) {
+                     float *out, int64_t ldo, const float *bias) {
     const unsigned gx = (unsigned)((C + 255) / 256), gy = (unsigned)((T + SQ_CONV_CHUNK - 1) / SQ_CONV_CHUNK);
-    hipLaunchKernelGGL(sq_conv_kernel, dim3(gx, gy), dim3(256), 0, st, step, (long long)tail_off, in, (long long)ldi, w, taps, mode, (long long)C, T, out, (long long)ldo);
+    hipLaunchKernelGGL(sq_conv_kernel, dim3(gx, gy), dim3(256), 0, st, step, (long long)tail_off, in, (long long)ldi, w, taps, mode, (long long)C, T, out, (long long)ldo, bias);
     if (gy > 1 && taps > 1) hipLaunchKernelGGL(sq_conv_tail_kernel, dim3(gx), dim3(256), 0, st, step, (long long)tail_off, in, (long long)ldi, taps, (long long)C, T);
 }
 
@@ -494,6 +494,166 @@ void psk_headnorm_gate(hipStream_t st, float *o, int64_t ldo, const float *g, in
     hipLaunchKernelGGL(sq_headnorm_gate_kernel, dim3(T, H), dim3(64), 0, st, o, (long long)ldo, g, (long long)ldg, w, w_stride, eps, dv);
 }
 
+
+// ---------------------------------------------------------------------------------------------------- state-space scan (Mamba-2)
+// S [N][P] per head with ONE decay per head and token: S <- g S + B (dt x)^T, o = S^T C + skip x, g = exp(-exp(a_log) dt), dt = softplus(dtraw + dt_bias); B and C belong to a
+// group of heads.  As above a column (one of P) evolves on its own and is spread over R lanes of 16 rows; here the state is kept column by column ([H][P][N]), so a lane's rows
+// are four 16-byte pieces and a column's lanes read one run.  A lane carries NC columns (cpb apart), so that B and C come out of LDS once for all of them.
+// LDS: cs, bs [TC][dp]; per token: g, dt
+template <int NC>
+__global__ __launch_bounds__(256) void sq_ssd_scan_kernel(const ps_seq_step *step, long long state_off, const float *x, const float *B, const float *C, long long ld,
+                                                          const float *dtraw, long long ldb, const float *a_log, const float *dt_bias, const float *skip, int H, int G, int N,
+                                                          int P, int R, int T, float *o, long long ldo) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    const int dp = SQ_NR * R, cpb = 256 / R;
+    float *cs = lds, *bs = cs + SQ_TC * dp, *gs = bs + SQ_TC * dp, *ds = gs + SQ_TC;
+    const int h = blockIdx.y, tid = threadIdx.x, s = tid % R, j0 = blockIdx.x * cpb * NC + tid / R;
+    const bool vec = N % 16 == 0; // (a lane's 16 rows are then all there or all not, and 16-byte aligned)
+    float *S0 = step->state + state_off + (long long)h * P * N;
+    float S[NC][SQ_NR];
+#pragma unroll
+    for (int c = 0; c < NC; c++) {
+        const int j = j0 + c * cpb;
+        const float *Sj = S0 + (long long)j * N + s * SQ_NR;
+        if (vec) {
+            const bool in = j < P && s * SQ_NR < N;
+#pragma unroll
+            for (int m4 = 0; m4 < SQ_NR / 4; m4++) {
+                const sq_f4 v = in ? *(const sq_f4 *)(Sj + 4 * m4) : sq_f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int e = 0; e < 4; e++) S[c][4 * m4 + e] = v[e];
+            }
+        } else {
+#pragma unroll
+            for (int m = 0; m < SQ_NR; m++) S[c][m] = (j < P && s * SQ_NR + m < N) ? Sj[m] : 0.f;
+        }
+    }
+    const long long nb = (long long)(h / (H / G)) * N, vb = (long long)h * P;
+    const float na = -expf(a_log[h]), db = dt_bias[h], sk = skip[h];
+    // the next round's inputs are requested before the current round's steps run
+    float pa[SQ_PF], pb[SQ_PF], pv[NC][SQ_TC], pd = 0.f;
+    auto fetch = [&](int t0) {
+        const int nt = min(SQ_TC, T - t0);
+#pragma unroll
+        for (int e = 0; e < SQ_PF; e++) {
+            const int i0 = tid + 256 * e, t = i0 / dp, i = i0 % dp;
+            const bool in = i0 < SQ_TC * dp && t < nt && i < N;
+            const long long at = (long long)(t0 + (in ? t : 0)) * ld + nb + (in ? i : 0);
+            pa[e] = in ? C[at] : 0.f;
+            pb[e] = in ? B[at] : 0.f;
+        }
+        if (tid < SQ_TC) pd = tid < nt ? dtraw[(long long)(t0 + tid) * ldb + h] : 0.f;
+#pragma unroll
+        for (int c = 0; c < NC; c++)
+#pragma unroll
+            for (int t = 0; t < SQ_TC; t++) pv[c][t] = (j0 + c * cpb < P && t < nt) ? x[(long long)(t0 + t) * ld + vb + j0 + c * cpb] : 0.f;
+    };
+    fetch(0);
+    for (int t0 = 0; t0 < T; t0 += SQ_TC) {
+        const int nt = min(SQ_TC, T - t0);
+        __syncthreads();
+#pragma unroll
+        for (int e = 0; e < SQ_PF; e++) {
+            const int i0 = tid + 256 * e;
+            if (i0 < SQ_TC * dp) {
+                cs[i0] = pa[e];
+                bs[i0] = pb[e];
+            }
+        }
+        if (tid < SQ_TC) { // (a token that is not there: g = 1, dt = 0 -- the state stays)
+            const float dt = tid < nt ? sq_softplus(pd + db) : 0.f;
+            ds[tid] = dt;
+            gs[tid] = expf(na * dt);
+        }
+        float xv[NC][SQ_TC];
+#pragma unroll
+        for (int c = 0; c < NC; c++)
+#pragma unroll
+            for (int t = 0; t < SQ_TC; t++) xv[c][t] = pv[c][t];
+        __syncthreads();
+        if (t0 + SQ_TC < T) fetch(t0 + SQ_TC);
+#pragma unroll
+        for (int t = 0; t < SQ_TC; t++) {
+            const sq_f4 *ct = (const sq_f4 *)(cs + t * dp + s * SQ_NR), *bt = (const sq_f4 *)(bs + t * dp + s * SQ_NR);
+            const float g = gs[t], dt = ds[t];
+            float u[NC], pp[NC][4];
+#pragma unroll
+            for (int c = 0; c < NC; c++) {
+                u[c] = dt * xv[c][t];
+#pragma unroll
+                for (int e = 0; e < 4; e++) pp[c][e] = 0.f;
+            }
+#pragma unroll
+            for (int m4 = 0; m4 < SQ_NR / 4; m4++) {
+                const sq_f4 c4 = ct[m4], b4 = bt[m4];
+#pragma unroll
+                for (int c = 0; c < NC; c++)
+#pragma unroll
+                    for (int e = 0; e < 4; e++) {
+                        S[c][4 * m4 + e] = fmaf(g, S[c][4 * m4 + e], b4[e] * u[c]);
+                        pp[c][e] = fmaf(c4[e], S[c][4 * m4 + e], pp[c][e]);
+                    }
+            }
+#pragma unroll
+            for (int c = 0; c < NC; c++) {
+                const float p = sq_col_sum((pp[c][0] + pp[c][1]) + (pp[c][2] + pp[c][3]), R);
+                if (j0 + c * cpb < P && s == 0 && t < nt) o[(long long)(t0 + t) * ldo + vb + j0 + c * cpb] = fmaf(sk, xv[c][t], p);
+            }
+        }
+    }
+#pragma unroll
+    for (int c = 0; c < NC; c++) {
+        const int j = j0 + c * cpb;
+        float *Sj = S0 + (long long)j * N + s * SQ_NR;
+        if (vec) {
+            if (j < P && s * SQ_NR < N) {
+#pragma unroll
+                for (int m4 = 0; m4 < SQ_NR / 4; m4++) *(sq_f4 *)(Sj + 4 * m4) = sq_f4{S[c][4 * m4], S[c][4 * m4 + 1], S[c][4 * m4 + 2], S[c][4 * m4 + 3]};
+            }
+        } else {
+#pragma unroll
+            for (int m = 0; m < SQ_NR; m++)
+                if (j < P && s * SQ_NR + m < N) Sj[m] = S[c][m];
+        }
+    }
+}
+void psk_ssd_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, const float *x, const float *B, const float *C, int64_t ld, const float *dtraw, int64_t ldb,
+                  const float *a_log, const float *dt_bias, const float *skip, int H, int G, int N, int P, int T, float *o, int64_t ldo) {
+    const int R = sq_lanes_per_col(N), cpb = 256 / R;
+    const size_t lds = (size_t)(2 * SQ_TC * SQ_NR * R + 2 * SQ_TC) * 4;
+    const bool two = T > SQ_TC && P > cpb;
+    const auto kernel = two ? sq_ssd_scan_kernel<2> : sq_ssd_scan_kernel<1>;
+    const int cols = two ? 2 * cpb : cpb;
+    hipLaunchKernelGGL(kernel, dim3((P + cols - 1) / cols, H), dim3(256), lds, st, step, (long long)state_off, x, B, C, (long long)ld, dtraw, (long long)ldb, a_log, dt_bias, skip,
+                       H, G, N, P, R, T, o, (long long)ldo);
+}
+
+// o <- o silu(z), then each of gridDim.y equal parts (n numbers) divided by its own root mean square, times w: block (token, part); a thread re-reads only what it wrote
+__global__ __launch_bounds__(1024) void sq_gate_partnorm_kernel(float *o, long long ldo, const float *z, long long ldz, const float *w, float eps, int n) {
+    __shared__ float red[16];
+    const int tid = threadIdx.x, nt = blockDim.x;
+    float *op = o + (long long)blockIdx.x * ldo + (long long)blockIdx.y * n;
+    const float *zp = z + (long long)blockIdx.x * ldz + (long long)blockIdx.y * n;
+    w += (long long)blockIdx.y * n;
+    float s = 0.f;
+    for (int i = tid; i < n; i += nt) {
+        const float v = op[i] * sq_silu(zp[i]);
+        op[i] = v;
+        s += v * v;
+    }
+#pragma unroll
+    for (int x = 32; x > 0; x >>= 1) s += __shfl_xor(s, x, 64);
+    if ((tid & 63) == 0) red[tid >> 6] = s;
+    __syncthreads();
+    float total = 0.f;
+    for (int k = 0; k < (nt >> 6); k++) total += red[k];
+    const float inv = 1.f / sqrtf(total / (float)n + eps);
+    for (int i = tid; i < n; i += nt) op[i] = op[i] * inv * w[i];
+}
+void psk_gate_partnorm(hipStream_t st, float *o, int64_t ldo, const float *z, int64_t ldz, const float *w, int parts, float eps, int64_t n, int T) {
+    const int pn = (int)(n / parts);
+    hipLaunchKernelGGL(sq_gate_partnorm_kernel, dim3(T, parts), dim3(T <= 8 && pn >= 1024 ? 1024 : 256), 0, st, o, (long long)ldo, z, (long long)ldz, w, eps, pn);
+}
 
 // ---------------------------------------------------------------------------------------------------- element-wise gated recurrence (minGRU)
 // y[t] = [ z | u | g ] pre-activations (C each, row stride ldy).  Per channel  a_t = 1 - sigmoid(z_t),  b_t = sigmoid(z_t) cand(u_t)  with

@@ -25,11 +25,12 @@ static __device__ __forceinline__ const float *la_row(const la_src &s, long long
 
 // qs: this wave's 16 rows in LDS, row stride qld floats, [DK1 | DK2]; pt: its 16 x 17 patch.  Accumulator row i of this lane (rows 4 (l / 16) + i)
 // sees key j when rowlo[i] <= j < rowhi[i] (a row that does not exist: rowhi = rowlo) and j < jend; j indexes whatever the sources hold (positions
-// of a window, blocks of a pooled store).  NJ: accumulator tiles (DV <= 16 NJ).
-template <int NJ>
+// of a window, rows of a store in front of it).  NJ: accumulator tiles (DV <= 16 NJ).  DIST: slope[i] * (qpos[i] - j) is taken off row i's score behind scale and soft cap.
+template <int NJ, bool DIST = false>
 static __device__ __forceinline__ void la_tile(const float *qs, int qld, float *pt, const la_src &k1, const la_src &k2, const la_src &vs, int DK1, int DK2, int DV,
                                                long long j0, long long jend, const long long (&rowlo)[4], const long long (&rowhi)[4], float scale, float (&m)[4], float (&l)[4],
-                                               la_f4 (&acc)[NJ], float softcap = 0.f) { // softcap > 0: score <- softcap tanh(score / softcap) behind the scale
+                                               la_f4 (&acc)[NJ], float softcap = 0.f, const float *slope = nullptr,
+                                               const long long *qpos = nullptr) { // softcap > 0: score <- softcap tanh(score / softcap) behind the scale
     const int lane = threadIdx.x & 63, lr = lane & 15, lq = lane >> 4;
     const long long jk = j0 + lr < jend ? j0 + lr : jend - 1; // (a key row that exists; masked below)
     la_f4 s4 = {0.f, 0.f, 0.f, 0.f};
@@ -61,6 +62,7 @@ static __device__ __forceinline__ void la_tile(const float *qs, int qld, float *
         const bool vis = j < jend && j >= rowlo[i] && j < rowhi[i];
         float sv = s4[i] * scale;
         if (softcap > 0.f) sv = softcap * tanhf(sv / softcap);
+        if constexpr (DIST) sv -= slope[i] * (float)(qpos[i] - j);
         const float s = vis ? sv : -INFINITY;
         float tm = s;
 #pragma unroll

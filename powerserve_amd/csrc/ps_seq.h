@@ -18,12 +18,14 @@ struct ps_seq_step {
     float *state;
     int32_t token0; // single-token steps: the token to embed (greedy decoding feeds its own arg-max back here)
     int32_t _pad;
+    int32_t prev, _pad2; // the token in front of the step's first one (a bigram embedding; meaningless at position 0)
 };
 
 enum { PSD_ACT_NONE = 0, PSD_ACT_XIELU = 1, PSD_ACT_TANH = 2,
        PSD_ACT_SILU_PAIR = 3,   // rows 2i / 2i + 1 of W are a gate and its partner: out[t][i] = silu(row 2i) * (row 2i + 1), N / 2 outputs (bias: one per row, added first)
        PSD_ACT_RELU_PAIR = 4,   // the same with relu on the gate
-       PSD_ACT_RELU2 = 5 };     // max(z, 0)^2
+       PSD_ACT_RELU2 = 5,       // max(z, 0)^2
+       PSD_ACT_SOFTCAP = 6 };   // act_p tanh(z / act_p)
 
 // out[t][n] = alpha * act(sum_k A(t, k) W[n][k] + bias[n]),  t < T
 //   A(t, k) = a[row(t)][k], row(t) = t, or (a_row0 + t) mod a_mod when a_mod > 0 (rows of a ring), or, where a_step is given, rows of the
@@ -63,7 +65,9 @@ struct psk_dense_args {
 int psk_dense(hipStream_t st, const psk_dense_args &a);
 void psk_dense_widen(hipStream_t st, const uint16_t *bf16, int64_t n, float *out);
 // out[t][:] = table[token(t)][:] * scale; tokens device int32 (step != NULL and T == 1: the token is step->token0)
-void psk_embed(hipStream_t st, const ps_dense *table, const int32_t *tokens, const ps_seq_step *step, int T, float scale, float *out, int64_t ldo);
+//   bigram given: + bigram[(prev * mul_prev + token * mul_cur) mod buckets][:], or its row `buckets` for position 0; prev = tokens[t - 1], in front of the step step->prev
+void psk_embed(hipStream_t st, const ps_dense *table, const int32_t *tokens, const ps_seq_step *step, int T, float scale, float *out, int64_t ldo, const ps_dense *bigram = nullptr,
+               int64_t buckets = 0, int64_t mul_prev = 0, int64_t mul_cur = 0);
 // out[r] = index of the first maximum of x[r][0..n)
 void psk_argmax_rows(hipStream_t st, const float *x, int64_t n, int rows, int32_t *out);
 
@@ -85,9 +89,9 @@ void psk_front(hipStream_t st, const float *src, int64_t stride, int nmix, const
 void psk_mingru_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, const float *y, int64_t ldy, int64_t C, int T, float *o, int64_t ldo);
 // Causal convolution over time on each channel, taps taken from the step's rows and, before them, from the sequence's tail (the last taps - 1
 // inputs of earlier steps, [taps - 1][C] at step->state + tail_off): out[t][c] = f(sum_j w[c][j] in(t - taps + 1 + j)[c]); mode 0: f = in(t) + sum
-// (a residual around the convolution), mode 1: f = silu(sum).  The tail is brought up to date behind it.
+// (a residual around the convolution), mode 1: f = silu(sum + bias[c]) (bias NULL: none).  The tail is brought up to date behind it.
 void psk_causal_conv(hipStream_t st, const ps_seq_step *step, int64_t tail_off, const float *in, int64_t ldi, const float *w, int taps, int mode,
-                     int64_t C, int T, float *out, int64_t ldo);
+                     int64_t C, int T, float *out, int64_t ldo, const float *bias = nullptr);
 // One token's sublayer boundary fused: x += norm_b(y) (y may be NULL), then h = conv(norm(x)) in the residual form with the tail update (wn may be NULL: stop after x);
 // hn (may be NULL) also receives norm(x) itself, for a sublayer that reads the unfiltered input
 void psk_boundary1(hipStream_t st, const ps_seq_step *step, float *x, const float *y, const float *wb, const float *wn, const float *cw, int taps, int64_t tail_off,
@@ -109,67 +113,81 @@ void psk_gla_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, co
 // per head: g = exp(-exp(a_log) softplus(araw + dt_bias)), beta = sigmoid(braw); S = g S; u = beta (v - S^T k); S += k u^T; o = S^T q.
 void psk_delta_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, const float *q, const float *k, const float *v, const float *braw,
                     const float *araw, int64_t ld, int64_t ldb, const float *a_log, const float *dt_bias, int H, int KH, int d, int dv, int T, float *o, int64_t ldo);
+// state-space scan, one decay per head.  x [T][H*P], B / C [T][G*N] after convolution + silu (row stride ld), dtraw [T][H] (row stride ldb); state [H][P][N] fp32 (a column's N
+// numbers together).  Per head (group g = h / (H / G)): dt = softplus(dtraw + dt_bias), S <- exp(-exp(a_log) dt) S + dt B x^T, o = S^T C + skip x.
+void psk_ssd_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, const float *x, const float *B, const float *C, int64_t ld, const float *dtraw, int64_t ldb,
+                  const float *a_log, const float *dt_bias, const float *skip, int H, int G, int N, int P, int T, float *o, int64_t ldo);
+// o[t] = part_norm(o[t] * silu(z[t])) * w: the gate first, then each of `parts` equal stretches of n / parts divided by its own root mean square
+void psk_gate_partnorm(hipStream_t st, float *o, int64_t ldo, const float *z, int64_t ldz, const float *w, int parts, float eps, int64_t n, int T);
 // o[t][h][:] = o / sqrt(mean_j o^2 + eps) * w(h, :) * silu(g[t][h][:]);  w_stride = dv (a weight per head) or 0 (one shared by the heads)
 void psk_headnorm_gate(hipStream_t st, float *o, int64_t ldo, const float *g, int64_t ldg, const float *w, int w_stride, float eps, int H, int dv, int T);
 
 // ---- k_moe.hip
 // Router of a mixture of experts, fp32: scores = sigmoid(router h[t]), or (softmax) the soft-max over all `experts` rows; choice scores = scores + correction (NULL: none);
 // with n_groups > 0 only rows of the `keep` groups (equal runs of neighbours) with the largest best choice score stay in the race; the `top` largest choice scores
-// (ties: the lower index) -> sel[t top + i], wgt[t top + i] (their SCORES, divided by their sum where norm_top); sgate[t] = sigmoid(shared_gate . h[t]) where given.
+// (ties: the lower index) -> sel[t top + i], wgt[t top + i] (their SCORES, divided by their sum where norm_top, times scale); sgate[t] = sigmoid(shared_gate . h[t]) where given.
 void psk_moe_route(hipStream_t st, const float *h, int64_t ldh, const float *router, const float *shared_gate, int experts, int top, int norm_top, int64_t K, int T,
-                   int32_t *sel, float *wgt, float *sgate, int softmax = 0, const float *correction = nullptr, int n_groups = 0, int keep = 0);
+                   int32_t *sel, float *wgt, float *sgate, int softmax = 0, const float *correction = nullptr, int n_groups = 0, int keep = 0, float scale = 1.f);
 // The S slots sorted by expert: seg [experts + 1] (slots of expert e are list[seg[e] .. seg[e + 1])), list [S]
 void psk_moe_plan(hipStream_t st, const int32_t *sel, int S, int experts, int32_t *seg, int32_t *list);
-// x[t] += alpha * sum_i (y[t top + i], or, for a slot whose sel >= n_real (an identity expert), wgt[slot] * h[t]);  y NULL: only the identity slots; sel NULL: only y
+// x[t] += alpha * sum_i (y[t top + i], or, for a slot whose sel >= n_real (an identity expert), wgt[slot] * h[t]);  y NULL: only the identity slots; sel NULL: only y; store: x[t] = instead of +=
 void psk_moe_combine(hipStream_t st, float *x, const float *y, int top, float alpha, int64_t n, int T, const int32_t *sel = nullptr, const float *wgt = nullptr,
-                     int n_real = 0, const float *h = nullptr, int64_t ldh = 0);
+                     int n_real = 0, const float *h = nullptr, int64_t ldh = 0, int store = 0);
 
 // ---- k_latent.hip
 // One token per block.  y[t] = [ dq (q_rank) | ckv (kv_rank) | kr (rot_dim) ]:  cq[t] = rmsnorm(dq) * qnorm;  ring row (pos mod cap):
-// c = rmsnorm(ckv) * kvnorm, kr with its first rot_dims numbers rotated at pos (pairs (i, i + rot_dims/2), angle pos * freq[i]).  Ring at step->state + ring_off: [cap][kv_rank + rot_dim].
+// c = rmsnorm(ckv) * kvnorm, kr with its first rot_dims numbers rotated at pos (angle of pair i: pos * freq[i]; pairs after `pairing`, a ps_rot_pairing, the same in all launches of a mixer).  Ring at step->state + ring_off: [cap][kv_rank + rot_dim].
 void psk_latent_prep(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, const float *y, int64_t ldy, const float *qnorm, const float *kvnorm,
                      float eps, int q_rank, int kv_rank, int rot_dim, int rot_dims, const float *freq, int T, float *cq, int64_t ldcq,
-                     float rot_mag = 1.f); // cos and sin of every rotation of this mixer are multiplied by rot_mag (the same value in all its launches); q_rank 0: no query latent
+                     float rot_mag = 1.f, int pairing = PS_ROT_HALVES); // cos and sin of every rotation of this mixer are multiplied by rot_mag (the same value in all its launches); q_rank 0: no query latent
 // Windowed soft-max attention over expanded keys / values.  q [T][H*(d+dr)] (rotated part not yet rotated), kv [Nw][H*d + H*dv] for the positions
 // first .. first + Nw - 1 where first = max(0, pos0 - window + 1) (the caller expands exactly these ring rows), rotated key parts from the ring.
 void psk_latent_attn(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, const float *q, int64_t ldq, const float *kv, int64_t ldkv,
                      const float *freq, int H, int d, int dr, int rot_dims, int dv, int kv_rank, int window, float scale, int T, float *o, int64_t ldo,
-                     float rot_mag = 1.f, const float *gate = nullptr, int64_t ldg = 0); // gate [T][H] raw: head h of token t times sigmoid(gate[t][h]) (all forms)
+                     float rot_mag = 1.f, const float *gate = nullptr, int64_t ldg = 0, int pairing = PS_ROT_HALVES); // gate [T][H] raw: head h of token t times sigmoid(gate[t][h]) (all forms)
 // The same attention on the matrix cores (fp32 MFMA), 16 tokens of a head per wave; _ok: the sizes it takes (d, dr multiples of 16, dv of 4, dv <= 128).
 bool psk_latent_attn_mfma_ok(int d, int dr, int dv);
 void psk_latent_attn_mfma(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, const float *q, int64_t ldq, const float *kv, int64_t ldkv,
                           const float *freq, int H, int d, int dr, int rot_dims, int dv, int kv_rank, int window, float scale, int T, float *o, int64_t ldo,
-                          float rot_mag = 1.f, const float *gate = nullptr, int64_t ldg = 0);
+                          float rot_mag = 1.f, const float *gate = nullptr, int64_t ldg = 0, int pairing = PS_ROT_HALVES);
 // Single-token step in the absorbed form: nothing is expanded per key, the ring's latents are keys and values for all heads at once.
 // q [H][d + dr] (row stride qstride, rotated part not yet rotated) -> o [H * dv].  ukv: rows uk | uv.  _ok: kv_rank, dr multiples of 16, kv_rank <= 512.
 bool psk_latent_absorbed_ok(int d, int dr, int dv, int R);
 size_t psk_latent_absorbed_scratch(int H, int R, int window);
 void psk_latent_absorbed(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, const float *q, int qstride, const ps_dense *ukv, const float *freq,
                          int H, int d, int dr, int rot_dims, int dv, int R, int window, float scale, float *scratch, float *o, float rot_mag = 1.f,
-                         const float *gate = nullptr);
+                         const float *gate = nullptr, int pairing = PS_ROT_HALVES);
 
 // ---- k_winattn.hip
+// What a token sees in front of its window comes from a second store with the ring's row layout at step->state + off: one row per POOLED BLOCK (pool > 0), or the rows of the
+// sequence's FIRST tokens (keep > 0: row = position; visible are those not in the window themselves), never both.  slope [H] (NULL: none): slope[h] * (query position - key
+// position) is taken off a score behind scale and soft cap (no pooled blocks).
+struct psk_front_store {
+    int64_t off = 0;
+    int pool = 0, keep = 0;
+};
 // y[t] = [ q (H d) | k (G d) | v (G dv) | ... ]: RMS norms over the whole q / k projections (qnorm / knorm, NULL: none), rotation of the first rot_dims numbers of
 // every head at the token's position (pairing: ps_rot_pairing; angle of pair i: pos * freq[i]); q -> q[t], k and v -> the ring row pos mod cap ([G d | G dv], ring at
-// step->state + ring_off); then the block means ([block][G d | G dv] at step->state + pool_off, pool > 0) are brought up to date.
-void psk_winattn_prep(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, int64_t pool_off, int pool, const float *y, int64_t ldy, const float *qnorm,
+// step->state + ring_off) and, for the first fs.keep positions, the front store; then the block means (fs.pool > 0) are brought up to date.  G 0: queries only.
+void psk_winattn_prep(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, psk_front_store fs, const float *y, int64_t ldy, const float *qnorm,
                       const float *knorm, float eps, int H, int G, int d, int dv, int rot_dims, int pairing, const float *freq, int T, float *q, int64_t ldq,
                       float qt_coef = 0.f, int qt_every = 0, // qt_every > 0: q[t] times 1 + qt_coef ln(floor((pos + 1) / qt_every) + 1)
                       int head_norm = 0, // 1: qnorm / knorm are [d] and the norms are taken per head
                       int v_unit = 0);   // 1: every head's value divided by its own root mean square
-// o[t][h] = gate(t, h) * soft-max attention of q[t][h] over the visible block means and the window's ring rows, scores times scale * temp[h], exp(sink[h]) in the
+// o[t][h] = gate(t, h) * soft-max attention of q[t][h] over the visible front store and the window's ring rows, scores times scale * temp[h], exp(sink[h]) in the
 // denominator; gate [T][..] raw (sigmoid here; column h, row stride ldg), temp / sink / gate may be NULL.
-void psk_winattn(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, int64_t pool_off, int pool, const float *q, int64_t ldq, const float *gate,
+void psk_winattn(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, psk_front_store fs, const float *q, int64_t ldq, const float *gate,
                  int64_t ldg, const float *temp, const float *sink, int H, int G, int d, int dv, int window, float scale, int T, float *o, int64_t ldo,
                  float softcap = 0.f, // softcap > 0 (all three forms): score <- softcap tanh(score / softcap) behind scale and temperature
-                 int gate_elem = 0);  // 1 (all three forms): gate [T][H dv], one sigmoid per output element instead of one per head
+                 int gate_elem = 0,   // 1 (all three forms): gate [T][H dv], one sigmoid per output element instead of one per head
+                 const float *slope = nullptr);
 // The same attention on the fp32 matrix cores for a portion, 16 tokens of a head per wave; _ok: the sizes it takes (d a multiple of 16, dv of 4, dv <= 128).
 bool psk_winattn_mfma_ok(int d, int dv);
-void psk_winattn_mfma(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, int64_t pool_off, int pool, const float *q, int64_t ldq, const float *gate,
+void psk_winattn_mfma(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, psk_front_store fs, const float *q, int64_t ldq, const float *gate,
                       int64_t ldg, const float *temp, const float *sink, int H, int G, int d, int dv, int window, float scale, int T, float *o, int64_t ldo,
-                      float softcap = 0.f, int gate_elem = 0);
+                      float softcap = 0.f, int gate_elem = 0, const float *slope = nullptr);
 // A single token on the matrix cores: rows = the heads of a key / value group, the keys spread over waves, partials merged in a second launch (same sizes).
-size_t psk_winattn_step_scratch(int H, int dv, int window, int pool, int64_t max_context);
-void psk_winattn_step(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, int64_t pool_off, int pool, const float *q, const float *gate, const float *temp,
+size_t psk_winattn_step_scratch(int H, int dv, int window, psk_front_store fs, int64_t max_context);
+void psk_winattn_step(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, psk_front_store fs, const float *q, const float *gate, const float *temp,
                       const float *sink, int H, int G, int d, int dv, int window, float scale, int64_t max_context, float *scratch, float *o, float softcap = 0.f,
-                      int gate_elem = 0);
+                      int gate_elem = 0, const float *slope = nullptr);

@@ -14,6 +14,9 @@
 // The feed-forward may be a mixture of experts: the router (fp32) picks per token, the experts' products are grouped launches of the dense kernels.
 // A PRE-NORM layer is  x += mixer(norm1(x)); x += ff(norm2(x)):  no filter, nothing normed behind a sublayer, the second norm reads what the mixer left; its norms
 // (and the final one) may be layer norms (norm_center).
+// A POST-NORM layer is  x += norm1b(mixer(x)); x += norm2b(ff(x)):  the sublayers read the residual stream itself and only what they put out is normed.
+// Attention layers may share keys and values: a layer with kv_from appends nothing and reads the ring (and the first tokens' rows) of the layer it names, which is sized for
+// the widest of its readers.  With a bigram embedding the last token of a portion is part of the slot's state.
 #include "ps_seq.h"
 
 #include <cmath>
@@ -29,7 +32,9 @@ struct LayerPlan { // one layer RUN (and, as `side`, the second mixer of one)
     int layer = 0; // index into the descriptor's layers (runs of a looped layer share it, and its weights)
     int64_t off_canon1 = 0, off_canon2 = 0, off_shift = 0, off_conv = 0, off_S = 0, off_ring = 0, off_pool = 0;
     int cap = 0;          // latent / windowed attention: ring rows
-    int64_t pool_rows = 0; // windowed attention: block means held
+    int64_t pool_rows = 0; // windowed attention: rows of the front store (block means, or the sequence's first tokens)
+    int32_t keep_rows = 0; // of these, first tokens the append writes
+    int owner = -1;        // windowed attention: the run whose ring and front store this one reads (-1: its own)
     float *freq = nullptr; // rot_dims / 2 angular frequencies (shared by the runs of a layer)
     float act_p = 0.f, act_q = 0.f;
     float rot_mag = 1.f; // latent: the factor on cos and sin that comes with frequency scaling by wavelength
@@ -73,14 +78,21 @@ struct ps_hip_seq {
     uint64_t weight_bytes = 0;
     std::vector<void *> owned;
     std::vector<ps_dense *> joints;
+    int64_t off_prev = -1; // bigram embedding: where a slot's state keeps the last token (an int32)
+    int32_t *prev_of(int slot) const { return off_prev < 0 ? nullptr : (int32_t *)(slot_state[slot] + off_prev); }
 };
 
-__global__ void seq_set_step_kernel(ps_seq_step *s, long long pos0, int n, int slot, float *state, int token0) {
+// last: the step's last token; prev (NULL: not kept): the slot's memory of the token before
+__global__ void seq_set_step_kernel(ps_seq_step *s, long long pos0, int n, int slot, float *state, int token0, int last, int32_t *prev) {
     s->pos0 = pos0; s->n = n; s->slot = slot; s->state = state; s->token0 = token0; s->_pad = 0;
+    s->prev = prev ? *prev : 0; s->_pad2 = 0;
+    if (prev) *prev = last;
 }
 // behind a greedy single-token step: the arg-max becomes the next token, the position moves on, the id is kept at ids[_pad++]
-__global__ void seq_advance_kernel(ps_seq_step *s, const int32_t *amax, int32_t *ids) {
+__global__ void seq_advance_kernel(ps_seq_step *s, const int32_t *amax, int32_t *ids, int32_t *prev) {
     const int32_t id = amax[0];
+    s->prev = s->token0;
+    if (prev) *prev = s->token0;
     ids[s->_pad] = id;
     s->_pad += 1;
     s->token0 = id;
@@ -112,6 +124,13 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
     m->groups = desc->norm_groups > 0 ? desc->norm_groups : 1;
     if (W % m->groups) return fail("norm_groups does not divide the width");
     int64_t moe_slots = 0, moe_experts = 0, moe_top = 1;
+    if (desc->bigram) {
+        const int64_t most = (int64_t)1 << 62;
+        if (desc->bigram_buckets <= 0 || desc->bigram->N != desc->bigram_buckets + 1 || desc->bigram->K != W || desc->bigram->dtype != desc->embed->dtype) return fail("bigram table shape");
+        if (desc->bigram_mul_prev < 0 || desc->bigram_mul_cur < 0 || (double)(desc->bigram_mul_prev) * desc->vocab + (double)(desc->bigram_mul_cur) * desc->vocab >= (double)most)
+            return fail("bigram multipliers");
+        m->off_prev = off; off += 4;
+    }
     bool depth = false;
     std::vector<int> order; // layer index of every run
     {
@@ -186,13 +205,16 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
                 return at + "windowed attention sizes (heads a multiple of kv_heads, vdim <= 256, even rot_dims <= dim)";
             if (l.rot_pairing != PS_ROT_HALVES && l.rot_pairing != PS_ROT_NEIGHBOURS) return at + "rot_pairing";
             if (l.gated < 0 || l.gated > 2) return at + "gated: 0 (none), 1 (a row per head) or 2 (a row per output element)";
-            P.ncat = H * d + G * d + G * dv + (l.gated == 2 ? H * dv : l.gated ? H : 0);
+            if (l.keep_first < 0 || (l.pool > 0 && (l.keep_first > 0 || l.dist_slope))) return at + "first tokens and distance slopes are not built together with pooled blocks";
+            if (l.kv_from < 0 || (l.kv_from > 0 && (desc->loop_times > 1 || l.kv_from > P.layer || l.pool > 0))) return at + "kv_from names an earlier layer (no loop, no pooled blocks)";
+            P.ncat = H * d + (l.kv_from > 0 ? 0 : G * d + G * dv) + (l.gated == 2 ? H * dv : l.gated ? H : 0);
             if (!shape(l.in_cat, P.ncat, W) || !shape(l.out, W, H * dv)) return at + "windowed attention tensors";
             if (l.pool > 0 || l.window <= 0 || l.window > m->max_context) m->needs_context = true;
             const int64_t window = l.window > 0 ? std::min<int64_t>(l.window, m->max_context) : m->max_context;
             P.d.window = (int32_t)window;
             P.cap = (int)(window - 1 + B);
-            P.pool_rows = l.pool > 0 ? m->max_context / l.pool + 1 : 0;
+            P.keep_rows = P.d.keep_first = (int32_t)std::min<int64_t>(l.keep_first, m->max_context);
+            P.pool_rows = l.pool > 0 ? m->max_context / l.pool + 1 : P.keep_rows;
             n1 = std::max(n1, P.ncat);
             n2 = std::max(n2, H * d);
             n3 = std::max(n3, H * dv);
@@ -208,6 +230,20 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
             n2 = std::max(n2, H * d);
             n3 = std::max(n3, H * dv);
             m->weight_bytes += dense_bytes(l.in_cat) + dense_bytes(l.decay2) + dense_bytes(l.out);
+        } else if (l.kind == PS_MIX_SSD) {
+            const int64_t G = l.kv_heads, inner = H * dv;
+            if (d > 256) return at + "state-space recurrence: state > 256 is not supported by the scan kernel";
+            if (G <= 0 || H % G || dv <= 0 || l.conv_taps < 1 || l.norm_parts <= 0 || inner % l.norm_parts) return at + "state-space sizes (heads a multiple of groups, norm_parts divides heads * vdim)";
+            P.cqkv = inner + 2 * G * d;
+            P.ncat = inner + P.cqkv + H;
+            if (!shape(l.in_cat, P.ncat, W) || !shape(l.out, W, inner) || !l.conv || !l.conv_bias || !l.a_log || !l.dt_bias || !l.skip || !l.onorm) return at + "state-space tensors";
+            P.off_conv = off; off += (int64_t)(l.conv_taps - 1) * P.cqkv;
+            off = (off + 3) / 4 * 4; // (16-byte pieces of the state)
+            P.off_S = off; off += inner * d;
+            n1 = std::max(n1, P.ncat);
+            n2 = std::max(n2, P.cqkv);
+            n3 = std::max(n3, inner);
+            m->weight_bytes += dense_bytes(l.in_cat) + dense_bytes(l.out);
         } else if (l.kind == PS_MIX_MINGRU) {
             P.ncat = 3 * d;
             if (!shape(l.in_cat, P.ncat, W) || !shape(l.out, W, d)) return at + "gated recurrence tensors";
@@ -227,10 +263,12 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
         P.d = desc->layers[P.layer];
         const ps_seq_layer &l = P.d;
         const std::string at = "layer " + std::to_string(P.layer) + ": ";
-        if (l.form != PS_LAYER_SEQUENTIAL && l.form != PS_LAYER_PARALLEL && l.form != PS_LAYER_PRENORM) return fail(at + "unknown layer form");
+        if (l.form != PS_LAYER_SEQUENTIAL && l.form != PS_LAYER_PARALLEL && l.form != PS_LAYER_PRENORM && l.form != PS_LAYER_POSTNORM) return fail(at + "unknown layer form");
+        if (l.form == PS_LAYER_POSTNORM && (l.norm1 || l.norm2 || l.canon1 || l.canon2 || l.depth_mix)) return fail(at + "a post-norm layer has no norm in front of a sublayer, no input filter and no depth average");
+        if (l.form == PS_LAYER_POSTNORM && (!l.norm1b || (l.ff_kind != PS_FF_NONE && !l.norm2b))) return fail(at + "output norm missing");
         if (l.form == PS_LAYER_PRENORM && (l.canon1 || l.canon2 || l.norm1b || l.norm2b || l.depth_mix)) return fail(at + "a pre-norm layer has no input filter, no norm behind a sublayer and no depth average");
         if (l.form != PS_LAYER_PRENORM && desc->norm_center) return fail(at + "layer norms (norm_center) are built for pre-norm layers");
-        if (!l.norm1 || (l.form == PS_LAYER_SEQUENTIAL && !l.norm1b) || (l.form == PS_LAYER_SEQUENTIAL && !l.canon1)) return fail(at + "norm / canon missing");
+        if ((!l.norm1 && l.form != PS_LAYER_POSTNORM) || (l.form == PS_LAYER_SEQUENTIAL && !l.norm1b) || (l.form == PS_LAYER_SEQUENTIAL && !l.canon1)) return fail(at + "norm / canon missing");
         if (l.canon1) { P.off_canon1 = off; off += (int64_t)(desc->canon_taps - 1) * W; }
         if (l.canon1 && (l.norm2 && l.form == PS_LAYER_PARALLEL)) return fail(at + "a parallel layer with an input filter has one norm");
         if (l.depth_mix) {
@@ -244,8 +282,8 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
             const bool moe = l.ff_kind == PS_FF_MOE_SWIGLU || l.ff_kind == PS_FF_MOE_RELU2;
             const int64_t pair = l.ff_kind == PS_FF_MOE_RELU2 ? 1 : 2; // rows of the up matrix per inner unit (a gate and its partner, or one)
             if (moe) {
-                if ((l.form != PS_LAYER_PARALLEL && l.form != PS_LAYER_PRENORM) || l.canon1)
-                    return fail(at + "a mixture of experts needs a parallel or pre-norm layer without an input filter");
+                if (l.form == PS_LAYER_SEQUENTIAL || l.canon1)
+                    return fail(at + "a mixture of experts needs a parallel, pre-norm or post-norm layer without an input filter");
                 const int rows = l.experts + l.moe_identity; // what the router puts out
                 if (l.experts <= 0 || l.moe_identity < 0 || l.top <= 0 || l.top > rows || l.ff <= 0 || !l.router) return fail(at + "mixture-of-experts sizes / router");
                 if (l.moe_groups > 0 && (rows % l.moe_groups || l.moe_keep <= 0 || l.moe_keep > l.moe_groups || l.top > (int64_t)l.moe_keep * (rows / l.moe_groups)))
@@ -279,12 +317,24 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
             P.side = std::make_shared<LayerPlan>();
             P.side->layer = P.layer;
             P.side->d = *l.beside;
+            if (P.side->d.kv_from > 0 || P.d.kv_from > 0) return fail(at + "kv_from is for a mixer on its own");
             if (P.side->d.beside) return fail(at + "a mixer beside another has none beside itself");
             e = plan_mixer(*P.side, at + "second mixer: ");
             if (!e.empty()) return fail(e);
         }
     }
     n2 = std::max(n2, m->n_t2q + nq);
+    for (auto &P : m->L) { // readers of another layer's keys: the owner's ring holds the widest reader's window, its front store the most first tokens
+        if (P.d.kind != PS_MIX_WINATTN || P.d.kv_from <= 0) continue;
+        LayerPlan &O = m->L[P.d.kv_from - 1]; // (no loop: a run is a layer)
+        const std::string at = "layer " + std::to_string(P.layer) + ": ";
+        if (O.d.kind != PS_MIX_WINATTN || O.d.kv_from > 0 || O.d.pool > 0 || O.side) return fail(at + "kv_from names a layer without keys of its own");
+        if (O.d.kv_heads != P.d.kv_heads || O.d.dim != P.d.dim || O.d.vdim != P.d.vdim) return fail(at + "kv_from: key / value heads, dim or vdim differ");
+        P.owner = P.d.kv_from - 1;
+        O.cap = std::max(O.cap, P.cap);
+        O.keep_rows = std::max(O.keep_rows, P.keep_rows);
+        O.pool_rows = O.keep_rows;
+    }
     if (depth)
         for (auto &P : m->L)
             if (P.d.form != PS_LAYER_PARALLEL || P.d.canon1) return fail("depth_mix needs every layer parallel and without an input filter");
@@ -294,12 +344,14 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
     };
     mixers([&](LayerPlan &P) {
         if (P.d.kind == PS_MIX_LATENT) { off = (off + 3) / 4 * 4; P.off_ring = off; off += (int64_t)P.cap * (P.d.kv_rank + P.d.rot_dim); } // (16-byte rows for the matrix-core kernels)
-        if (P.d.kind == PS_MIX_WINATTN) {
+        if (P.d.kind == PS_MIX_WINATTN && P.owner < 0) {
             const int64_t rs = (int64_t)P.d.kv_heads * (P.d.dim + P.d.vdim);
             off = (off + 3) / 4 * 4; P.off_ring = off; off += (int64_t)P.cap * rs;
             off = (off + 3) / 4 * 4; P.off_pool = off; off += P.pool_rows * rs;
         }
     });
+    for (auto &P : m->L)
+        if (P.owner >= 0) { const LayerPlan &O = m->L[P.owner]; P.off_ring = O.off_ring; P.off_pool = O.off_pool; P.cap = O.cap; }
     m->state_floats = off;
     auto alloc = [&](void **p, size_t bytes) {
         if (ps_dev_malloc(p, bytes + 256) != hipSuccess) return false;
@@ -383,7 +435,7 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
         size_t wb = 0;
         mixers([&](LayerPlan &P) {
             if (P.d.kind == PS_MIX_WINATTN && psk_winattn_mfma_ok(P.d.dim, P.d.vdim))
-                wb = std::max(wb, psk_winattn_step_scratch(P.d.heads, P.d.vdim, P.d.window, P.d.pool, m->max_context));
+                wb = std::max(wb, psk_winattn_step_scratch(P.d.heads, P.d.vdim, P.d.window, psk_front_store{P.off_pool, P.d.pool, P.d.keep_first}, m->max_context));
         });
         if (wb) ok = ok && alloc((void **)&m->win_scratch, wb);
     }
@@ -453,7 +505,8 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
     const int64_t W = D.width;
     const bool tiled = (m->mode & 2) != 0;
     const int64_t BW = (int64_t)D.max_batch * W;
-    psk_embed(st, D.embed, from_step ? nullptr : m->tokens, m->step, T, m->embed_scale, m->hist ? m->hist : m->x, W);
+    psk_embed(st, D.embed, from_step ? nullptr : m->tokens, m->step, T, m->embed_scale, m->hist ? m->hist : m->x, W, D.bigram, D.bigram_buckets, D.bigram_mul_prev,
+              D.bigram_mul_cur);
     auto mm = [&](const ps_dense *w, const float *a, int64_t lda, float *out, int64_t ldo) {
         psk_dense_args g;
         g.w = w; g.a = a; g.lda = lda; g.T = T; g.out = out; g.ldo = ldo; g.force_tiled = tiled; g.pack = m->pack; g.pack_bytes = m->pack_bytes;
@@ -471,40 +524,40 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
             psk_causal_conv(st, m->step, tail_off, m->hn, W, cw, D.canon_taps, 0, W, T, m->h, W);
         }
     };
-    // One mixer on the input m->h.  Its output projection writes m->y (into == NULL) or adds out_scale times its result to `into`.
-    auto mixer = [&](const LayerPlan &P, float *into, float out_scale) {
+    // One mixer on the input `in`.  Its output projection writes m->y (into == NULL) or adds out_scale times its result to `into`.
+    auto mixer = [&](const LayerPlan &P, const float *in, float *into, float out_scale) {
         const ps_seq_layer &l = P.d;
         const int64_t H = l.heads, d = l.dim, dv = l.vdim;
         float *t1 = m->t1 + P.in_off;                       // this mixer's columns of the (possibly joint) input projection
         const int64_t ld1 = P.in_ld ? P.in_ld : P.ncat;
         auto out_proj = [&](const float *a, int64_t lda) {
             auto g = mm(l.out, a, lda, into ? into : m->y, W);
-            g.alpha = out_scale; g.accum = into ? 1 : 0;
+            g.alpha = out_scale; g.accum = into ? 1 : 0; g.bias = l.out_bias;
             psk_dense(st, g);
         };
         if (l.kind == PS_MIX_WKV) {
             const int64_t Hd = H * d, NW = 5 * Hd;
             const ps_dense *ws[4] = {l.in_r, l.in_k, l.in_v, l.in_g};
             for (int s = 0; s < 4; s++) {
-                auto g = mm(ws[s], m->h, W, m->t1 + s * Hd, NW);
+                auto g = mm(ws[s], in, W, m->t1 + s * Hd, NW);
                 g.mu = l.mu + s * W; g.shift0 = state + P.off_shift;
                 psk_dense(st, g);
             }
             {
-                auto g = mm(l.decay1, m->h, W, m->t2, l.decay_rank);
+                auto g = mm(l.decay1, in, W, m->t2, l.decay_rank);
                 g.mu = l.mu + 4 * W; g.shift0 = state + P.off_shift; g.act = PSD_ACT_TANH;
                 psk_dense(st, g);
                 auto g2 = mm(l.decay2, m->t2, l.decay_rank, m->t1 + 4 * Hd, NW);
                 g2.bias = l.decay0;
                 psk_dense(st, g2);
             }
-            psk_state_store(st, m->step, P.off_shift, m->h + (int64_t)(T - 1) * W, W);
+            psk_state_store(st, m->step, P.off_shift, in + (int64_t)(T - 1) * W, W);
             psk_wkv_scan(st, m->step, P.off_S, m->t1, m->t1 + Hd, m->t1 + 2 * Hd, m->t1 + 4 * Hd, NW, l.bonus, (int)H, (int)d, T, m->t3, Hd);
             psk_headnorm_gate(st, m->t3, Hd, m->t1 + 3 * Hd, NW, l.onorm, (int)d, D.norm_eps, (int)H, (int)d, T);
             out_proj(m->t3, Hd);
         } else if (l.kind == PS_MIX_DELTA) {
             const int64_t KHd = (int64_t)l.kv_heads * d, Hv = H * dv;
-            if (!P.in_ld) psk_dense(st, mm(l.in_cat, m->h, W, t1, ld1));
+            if (!P.in_ld) psk_dense(st, mm(l.in_cat, in, W, t1, ld1));
             psk_causal_conv(st, m->step, P.off_conv, t1, ld1, l.conv, l.conv_taps, 1, P.cqkv, T, m->t2, P.cqkv);
             psk_delta_scan(st, m->step, P.off_S, m->t2, m->t2 + KHd, m->t2 + 2 * KHd, t1 + P.cqkv + Hv, t1 + P.cqkv + Hv + H, P.cqkv, ld1, l.a_log, l.dt_bias,
                            (int)H, l.kv_heads, (int)d, (int)dv, T, m->t3, Hv);
@@ -513,7 +566,7 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
         } else if (l.kind == PS_MIX_GLA) {
             // t1 = [ q | k | v | g | a1 ]; the decay's second matrix (with its bias) -> t2; scan -> t3; per-head norm and gate; out
             const int64_t Hd = H * d, Hv = H * dv;
-            if (!P.in_ld) psk_dense(st, mm(l.in_cat, m->h, W, t1, ld1));
+            if (!P.in_ld) psk_dense(st, mm(l.in_cat, in, W, t1, ld1));
             auto g2 = mm(l.decay2, t1 + 2 * Hd + 2 * Hv, ld1, m->t2, Hd);
             g2.bias = l.decay0;
             psk_dense(st, g2);
@@ -524,29 +577,40 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
             // t1 = [ q | k | v | gate ] (+ bias); norms, rotation, ring append and block means; attention -> t3; out
             const int64_t G = l.kv_heads, Hd = H * d, Hv = H * dv;
             if (!P.in_ld) {
-                auto g = mm(l.in_cat, m->h, W, t1, ld1);
+                auto g = mm(l.in_cat, in, W, t1, ld1);
                 g.bias = l.in_bias;
                 psk_dense(st, g);
             }
-            psk_winattn_prep(st, m->step, P.off_ring, P.cap, P.off_pool, l.pool, t1, ld1, l.qnorm, l.knorm, D.norm_eps, (int)H, (int)G, (int)d, (int)dv, l.rot_dims,
-                             l.rot_pairing, P.freq, T, m->t2, Hd, l.qtemp_coef, l.qtemp_every, l.head_norm, l.v_unit);
-            const float *gate = l.gated ? t1 + Hd + G * d + G * dv : nullptr;
+            const bool reads = P.owner >= 0; // (another layer's keys and values: queries only)
+            psk_winattn_prep(st, m->step, P.off_ring, P.cap, psk_front_store{P.off_pool, l.pool, reads ? 0 : P.keep_rows}, t1, ld1, l.qnorm, l.knorm, D.norm_eps, (int)H,
+                             reads ? 0 : (int)G, (int)d, (int)dv, l.rot_dims, l.rot_pairing, P.freq, T, m->t2, Hd, l.qtemp_coef, l.qtemp_every, l.head_norm, l.v_unit);
+            const psk_front_store fs{P.off_pool, l.pool, l.keep_first};
+            const float *gate = l.gated ? t1 + Hd + (reads ? 0 : G * d + G * dv) : nullptr;
             const int ge = l.gated == 2; // a gate per output element
             const bool mfma = (m->mode & 2) == 0 && (G * (d + dv)) % 4 == 0 && psk_winattn_mfma_ok((int)d, (int)dv);
             if (mfma && T == 1 && m->win_scratch)
-                psk_winattn_step(st, m->step, P.off_ring, P.cap, P.off_pool, l.pool, m->t2, gate, l.temp, l.sink, (int)H, (int)G, (int)d, (int)dv, l.window, l.scale,
-                                 m->max_context, m->win_scratch, m->t3, l.softcap, ge);
+                psk_winattn_step(st, m->step, P.off_ring, P.cap, fs, m->t2, gate, l.temp, l.sink, (int)H, (int)G, (int)d, (int)dv, l.window, l.scale,
+                                 m->max_context, m->win_scratch, m->t3, l.softcap, ge, l.dist_slope);
             else if (mfma)
-                psk_winattn_mfma(st, m->step, P.off_ring, P.cap, P.off_pool, l.pool, m->t2, Hd, gate, ld1, l.temp, l.sink, (int)H, (int)G, (int)d, (int)dv, l.window, l.scale,
-                                 T, m->t3, Hv, l.softcap, ge);
+                psk_winattn_mfma(st, m->step, P.off_ring, P.cap, fs, m->t2, Hd, gate, ld1, l.temp, l.sink, (int)H, (int)G, (int)d, (int)dv, l.window, l.scale,
+                                 T, m->t3, Hv, l.softcap, ge, l.dist_slope);
             else
-                psk_winattn(st, m->step, P.off_ring, P.cap, P.off_pool, l.pool, m->t2, Hd, gate, ld1, l.temp, l.sink, (int)H, (int)G, (int)d, (int)dv, l.window, l.scale, T,
-                            m->t3, Hv, l.softcap, ge);
+                psk_winattn(st, m->step, P.off_ring, P.cap, fs, m->t2, Hd, gate, ld1, l.temp, l.sink, (int)H, (int)G, (int)d, (int)dv, l.window, l.scale, T,
+                            m->t3, Hv, l.softcap, ge, l.dist_slope);
             out_proj(m->t3, Hv);
+        } else if (l.kind == PS_MIX_SSD) {
+            // t1 = [ z | x | B | C | dt ]; x, B and C through the convolution -> t2; scan -> t3; gate and norm; out
+            const int64_t inner = H * dv, GN = (int64_t)l.kv_heads * d;
+            if (!P.in_ld) psk_dense(st, mm(l.in_cat, in, W, t1, ld1));
+            psk_causal_conv(st, m->step, P.off_conv, t1 + inner, ld1, l.conv, l.conv_taps, 1, P.cqkv, T, m->t2, P.cqkv, l.conv_bias);
+            psk_ssd_scan(st, m->step, P.off_S, m->t2, m->t2 + inner, m->t2 + inner + GN, P.cqkv, t1 + inner + P.cqkv, ld1, l.a_log, l.dt_bias, l.skip, (int)H, l.kv_heads, (int)d,
+                         (int)dv, T, m->t3, inner);
+            psk_gate_partnorm(st, m->t3, inner, t1, ld1, l.onorm, l.norm_parts, D.norm_eps, inner, T);
+            out_proj(m->t3, inner);
         } else if (l.kind == PS_MIX_MINGRU) {
             // t1 = [ z | x | g ] (+ bias); the recurrence and the gate -> t3; out
             if (!P.in_ld) {
-                auto g = mm(l.in_cat, m->h, W, t1, ld1);
+                auto g = mm(l.in_cat, in, W, t1, ld1);
                 g.bias = l.in_bias;
                 psk_dense(st, g);
             }
@@ -559,14 +623,14 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
             float *cq = m->t2, *q = direct ? m->t1 : m->t2 + (int64_t)D.max_batch * m->n_t2q;
             const int64_t ldq = direct ? P.ncat : nq;
             const float *gate = l.gated ? m->t1 + P.ncat - H : nullptr;
-            psk_dense(st, mm(l.in_cat, m->h, W, m->t1, P.ncat));
+            psk_dense(st, mm(l.in_cat, in, W, m->t1, P.ncat));
             psk_latent_prep(st, m->step, P.off_ring, P.cap, direct ? m->t1 + nq : m->t1, P.ncat, l.qnorm, l.kvnorm, D.norm_eps, l.q_rank, l.kv_rank, (int)dr, l.rot_dims, P.freq, T,
-                            cq, l.q_rank, P.rot_mag);
+                            cq, l.q_rank, P.rot_mag, l.rot_pairing);
             if (!direct) psk_dense(st, mm(l.uq, cq, l.q_rank, q, nq));
             const bool plain = (m->mode & 2) != 0, rows4 = (l.kv_rank + dr) % 4 == 0 && l.kv_rank % 4 == 0;
             if (T == 1 && !plain && m->abs_scratch && psk_latent_absorbed_ok((int)d, (int)dr, (int)dv, l.kv_rank)) {
                 psk_latent_absorbed(st, m->step, P.off_ring, P.cap, q, (int)(d + dr), l.ukv, P.freq, (int)H, (int)d, (int)dr, l.rot_dims, (int)dv, l.kv_rank, l.window,
-                                    l.scale, m->abs_scratch, m->t3, P.rot_mag, gate);
+                                    l.scale, m->abs_scratch, m->t3, P.rot_mag, gate, l.rot_pairing);
             } else {
                 // the window's keys and values, expanded from the ring rows  max(0, pos0 - window + 1) .. pos0 + T - 1
                 auto g = mm(l.ukv, state + P.off_ring, rs, m->kvx, H * d + Hv);
@@ -575,17 +639,17 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
                 psk_dense(st, g);
                 if (!plain && rows4 && psk_latent_attn_mfma_ok((int)d, (int)dr, (int)dv))
                     psk_latent_attn_mfma(st, m->step, P.off_ring, P.cap, q, ldq, m->kvx, H * d + Hv, P.freq, (int)H, (int)d, (int)dr, l.rot_dims, (int)dv, l.kv_rank, l.window,
-                                         l.scale, T, m->t3, Hv, P.rot_mag, gate, P.ncat);
+                                         l.scale, T, m->t3, Hv, P.rot_mag, gate, P.ncat, l.rot_pairing);
                 else
                     psk_latent_attn(st, m->step, P.off_ring, P.cap, q, ldq, m->kvx, H * d + Hv, P.freq, (int)H, (int)d, (int)dr, l.rot_dims, (int)dv, l.kv_rank, l.window,
-                                    l.scale, T, m->t3, Hv, P.rot_mag, gate, P.ncat);
+                                    l.scale, T, m->t3, Hv, P.rot_mag, gate, P.ncat, l.rot_pairing);
             }
             out_proj(m->t3, Hv);
         }
     };
-    auto joint_in = [&](const LayerPlan &P) { // both mixers' stacked input projections in one product
+    auto joint_in = [&](const LayerPlan &P, const float *in) { // both mixers' stacked input projections in one product
         if (!P.joint) return;
-        auto g = mm(P.joint, m->h, W, m->t1, P.in_ld);
+        auto g = mm(P.joint, in, W, m->t1, P.in_ld);
         g.bias = P.joint_bias;
         psk_dense(st, g);
     };
@@ -598,17 +662,17 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
         if (l.ff_kind != PS_FF_DENSE_XIELU) g.bias = l.ff_up_bias;
         psk_dense(st, g);
     };
-    // The feed-forward of a parallel or pre-norm layer on `in`, added to xr times alpha.  Mixture of experts: slot s = t top + i is token t's i-th choice; the router's
+    // The feed-forward of a layer on `in`, added to xr times alpha (store: written there instead).  Mixture of experts: slot s = t top + i is token t's i-th choice; the router's
     // score scales what the expert READS (the A operand of its first product) or, moe_weight_output, what it puts out (the rows of its inner activation: the second
     // product is linear); a few tokens run grouped mat-vecs, a portion tiles over the slots sorted by expert.  A choice beyond the experts that have matrices is an
     // identity expert: no product touches its slot, and its weight times the input joins the sum.
-    auto feed_forward = [&](const LayerPlan &P, const float *in, float *xr, float alpha) {
+    auto feed_forward = [&](const LayerPlan &P, const float *in, float *xr, float alpha, bool store = false) {
         const ps_seq_layer &l = P.d;
         const bool moe = l.ff_kind == PS_FF_MOE_SWIGLU || l.ff_kind == PS_FF_MOE_RELU2;
         if (!moe) {
             ff_up(P, in);
             auto g = mm(l.ff_down, m->t4, l.ff, xr, W);
-            g.accum = 1; g.alpha = alpha;
+            g.accum = !store; g.alpha = alpha;
             if (l.ff_kind != PS_FF_DENSE_XIELU) g.bias = l.ff_down_bias;
             psk_dense(st, g);
             return;
@@ -616,7 +680,7 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
         const int E = l.experts, rows = E + l.moe_identity, top = l.top, S = T * top;
         const int act = l.ff_kind == PS_FF_MOE_RELU2 ? PSD_ACT_RELU2 : PSD_ACT_SILU_PAIR;
         psk_moe_route(st, in, W, l.router, l.shared_gate, rows, top, l.moe_norm_top, W, T, m->moe_sel, m->moe_wgt, m->moe_sg, l.moe_softmax, l.moe_correction, l.moe_groups,
-                      l.moe_keep);
+                      l.moe_keep, l.moe_scale != 0.f ? l.moe_scale : 1.f);
         const bool mv = !tiled && T <= 8 && (size_t)std::max<int64_t>(W, (int64_t)top * l.ff) * 4 + 64 <= 128 * 1024;
         if (!mv) psk_moe_plan(st, m->moe_sel, S, rows, m->moe_seg, m->moe_list);
         auto grouped = [&](psk_dense_args &g) {
@@ -636,14 +700,18 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
             auto g = mm(l.ff_down, m->t4, l.ff, xr, W);
             grouped(g);
             if (mv) {
-                g.T = T; g.g_inner = top; g.accum = 1; g.alpha = alpha;
+                g.T = T; g.g_inner = top; g.accum = !store; g.alpha = alpha;
                 if (l.moe_identity) { g.g_ident = in; g.g_ident_ld = W; g.g_ident_w = m->moe_wgt; summed = true; } // (the identity slots' share inside the same launch)
             }
-            else if (top == 1) { g.T = S; g.accum = 1; g.alpha = alpha; }
+            else if (top == 1) {
+                // (an identity expert's slot has no product: a store must find a zero there)
+                if (store && l.moe_identity) psk_fill(st, xr, 0.f, (int64_t)T * W);
+                g.T = S; g.accum = !store || l.moe_identity; g.alpha = alpha;
+            }
             else { g.T = S; g.out = m->moe_y; } // (two slots of a token sit in different tiles: per-slot results, summed below)
             psk_dense(st, g);
             if (!mv && top > 1) {
-                psk_moe_combine(st, xr, m->moe_y, top, alpha, W, T, l.moe_identity ? m->moe_sel : nullptr, m->moe_wgt, E, in, W);
+                psk_moe_combine(st, xr, m->moe_y, top, alpha, W, T, l.moe_identity ? m->moe_sel : nullptr, m->moe_wgt, E, in, W, store);
                 summed = true;
             }
         }
@@ -667,12 +735,22 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
         if (l.form == PS_LAYER_PRENORM) {
             // x += mixer(norm1(x)), then x += ff(norm2(x)): each sublayer's front is one launch, its output projection adds straight into the residual stream
             psk_front(st, m->x, 0, 1, nullptr, nullptr, nullptr, l.norm1, m->h, nullptr, nullptr, m->groups, D.norm_offset, D.norm_eps, W, T, D.norm_center);
-            joint_in(P);
-            mixer(P, m->x, l.mix_scale);
-            if (P.side) mixer(*P.side, m->x, P.side->d.mix_scale);
+            joint_in(P, m->h);
+            mixer(P, m->h, m->x, l.mix_scale);
+            if (P.side) mixer(*P.side, m->h, m->x, P.side->d.mix_scale);
             if (l.ff_kind != PS_FF_NONE) {
                 psk_front(st, m->x, 0, 1, nullptr, nullptr, nullptr, l.norm2, m->h, nullptr, nullptr, m->groups, D.norm_offset, D.norm_eps, W, T, D.norm_center);
                 feed_forward(P, m->h, m->x, 1.f);
+            }
+        } else if (l.form == PS_LAYER_POSTNORM) {
+            // x += norm_b(mixer(x)), then x += norm_b(ff(x)): a sublayer's first product reads the residual stream, its last one writes y
+            joint_in(P, m->x);
+            mixer(P, m->x, nullptr, l.mix_scale);
+            if (P.side) mixer(*P.side, m->x, m->y, P.side->d.mix_scale);
+            boundary(m->y, l.norm1b, nullptr, nullptr, 0);
+            if (l.ff_kind != PS_FF_NONE) {
+                feed_forward(P, m->x, m->y, 1.f, true);
+                boundary(m->y, l.norm2b, nullptr, nullptr, 0);
             }
         } else if (l.form == PS_LAYER_PARALLEL && !l.canon1) {
             // No input filter: one launch makes the layer's input (with depth_mix: the previous layer's average over X_0 .. X_li, kept as this layer's X to add
@@ -681,25 +759,25 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
             float *h2 = l.norm2 ? m->hn : nullptr;
             if (m->hist) psk_front(st, m->hist, BW, li + 1, li ? m->L[li - 1].d.depth_mix : nullptr, nullptr, xr, l.norm1, m->h, l.norm2, h2, m->groups, D.norm_offset, D.norm_eps, W, T);
             else psk_front(st, m->x, 0, 1, nullptr, nullptr, nullptr, l.norm1, m->h, l.norm2, h2, m->groups, D.norm_offset, D.norm_eps, W, T);
-            joint_in(P);
-            mixer(P, xr, res * l.mix_scale);
-            if (P.side) mixer(*P.side, xr, res * P.side->d.mix_scale);
+            joint_in(P, m->h);
+            mixer(P, m->h, xr, res * l.mix_scale);
+            if (P.side) mixer(*P.side, m->h, xr, res * P.side->d.mix_scale);
             if (l.ff_kind != PS_FF_NONE) feed_forward(P, h2 ? h2 : m->h, xr, res);
             if (m->dbg_layers && !any_pos && m->hist)
                 psk_front(st, m->hist, BW, li + 2, l.depth_mix, nullptr, m->dbg_layers + (int64_t)li * BW, nullptr, nullptr, nullptr, nullptr, 1, 0.f, D.norm_eps, W, T);
         } else if (l.form == PS_LAYER_PARALLEL) {
             // hn = norm(x), h = conv(hn); both mixers and the feed-forward add their output projections straight into the residual stream
             boundary(nullptr, nullptr, l.norm1, l.canon1, P.off_canon1);
-            joint_in(P);
-            mixer(P, m->x, res * l.mix_scale);
-            if (P.side) mixer(*P.side, m->x, res * P.side->d.mix_scale);
+            joint_in(P, m->h);
+            mixer(P, m->h, m->x, res * l.mix_scale);
+            if (P.side) mixer(*P.side, m->h, m->x, res * P.side->d.mix_scale);
             if (l.ff_kind != PS_FF_NONE) feed_forward(P, m->hn, m->x, res);
         } else {
             const bool summed = P.side != nullptr || l.mix_scale != 1.f;
             if (summed) psk_fill(st, m->y, 0.f, (int64_t)T * W);
-            joint_in(P);
-            mixer(P, summed ? m->y : nullptr, l.mix_scale);
-            if (P.side) mixer(*P.side, m->y, P.side->d.mix_scale);
+            joint_in(P, m->h);
+            mixer(P, m->h, summed ? m->y : nullptr, l.mix_scale);
+            if (P.side) mixer(*P.side, m->h, m->y, P.side->d.mix_scale);
             const bool nseq = next && next->d.form == PS_LAYER_SEQUENTIAL;
             const float *nn = nseq ? next->d.norm1 : nullptr, *nc = nseq ? next->d.canon1 : nullptr;
             const int64_t no = nseq ? next->off_canon1 : 0;
@@ -731,6 +809,7 @@ static void seq_head(ps_hip_seq *m, const int32_t *idx, int rows) {
     }
     psk_dense_args g;
     g.w = D.head; g.a = m->xn; g.lda = D.width; g.T = rows; g.out = m->logits; g.ldo = D.vocab; g.alpha = D.logit_scale; g.force_tiled = (m->mode & 2) != 0; g.pack = m->pack; g.pack_bytes = m->pack_bytes;
+    if (D.logit_softcap > 0.f) { g.act = PSD_ACT_SOFTCAP; g.act_p = D.logit_softcap; }
     psk_dense(st, g);
     psk_argmax_rows(st, m->logits, D.vocab, rows, m->amax);
 }
@@ -753,7 +832,8 @@ int ps_hip_seq_forward(ps_hip_seq *m, int slot, const int32_t *tokens, int n, co
         const int T = std::min(B, n - t0);
         const int64_t pos0 = m->slot_pos[slot];
         PS_CHECK(c, hipMemcpyAsync(m->tokens, tokens + t0, (size_t)T * 4, hipMemcpyHostToDevice, c->stream));
-        hipLaunchKernelGGL(seq_set_step_kernel, dim3(1), dim3(1), 0, c->stream, m->step, (long long)pos0, T, slot, m->slot_state[slot], (int)tokens[t0]);
+        hipLaunchKernelGGL(seq_set_step_kernel, dim3(1), dim3(1), 0, c->stream, m->step, (long long)pos0, T, slot, m->slot_state[slot], (int)tokens[t0], (int)tokens[t0 + T - 1],
+                           m->prev_of(slot));
         seq_layers(m, m->slot_state[slot], T, pos0, false, false);
         std::vector<int32_t> idx;
         const int w0 = wi;
@@ -787,11 +867,11 @@ int ps_hip_seq_decode_greedy(ps_hip_seq *m, int slot, int32_t token, int steps, 
         m->graphs.clear();
     }
     float *state = m->slot_state[slot];
-    hipLaunchKernelGGL(seq_set_step_kernel, dim3(1), dim3(1), 0, c->stream, m->step, (long long)m->slot_pos[slot], 1, slot, state, (int)token);
+    hipLaunchKernelGGL(seq_set_step_kernel, dim3(1), dim3(1), 0, c->stream, m->step, (long long)m->slot_pos[slot], 1, slot, state, (int)token, (int)token, m->prev_of(slot));
     auto one = [&]() {
         seq_layers(m, state, 1, 0, true, true);
         seq_head(m, nullptr, 1);
-        hipLaunchKernelGGL(seq_advance_kernel, dim3(1), dim3(1), 0, c->stream, m->step, m->amax, m->ids);
+        hipLaunchKernelGGL(seq_advance_kernel, dim3(1), dim3(1), 0, c->stream, m->step, m->amax, m->ids, m->prev_of(slot));
     };
     if (m->mode & 1) {
         for (int i = 0; i < steps; i++) one();
@@ -853,7 +933,7 @@ int ps_hip_seq_bench_kernel(ps_hip_seq *m, int which, int T, int reps, double *u
             for (int first = 0; first < (mv && P.d.moe_identity ? 64 : 1); first++) {
                 if (first && !embed_from(first)) return seq_fail(c, "seq_bench_kernel: embedding");
                 psk_moe_route(c->stream, m->h, W, P.d.router, P.d.shared_gate, rows, top, P.d.moe_norm_top, W, T, m->moe_sel, m->moe_wgt, m->moe_sg, P.d.moe_softmax,
-                              P.d.moe_correction, P.d.moe_groups, P.d.moe_keep);
+                              P.d.moe_correction, P.d.moe_groups, P.d.moe_keep, P.d.moe_scale != 0.f ? P.d.moe_scale : 1.f);
                 PS_CHECK(c, hipMemcpyAsync(sel.data(), m->moe_sel, (size_t)S * 4, hipMemcpyDeviceToHost, c->stream));
                 PS_CHECK(c, hipStreamSynchronize(c->stream));
                 bool all_real = true;

@@ -102,7 +102,9 @@ SeqLayer._fields_ = ([(n, C.c_int32) for n in ("kind", "heads", "kv_heads", "dim
                 [(n, C.c_void_p) for n in ("router", "shared_gate", "shared_up", "shared_down")] +
                 [("head_norm", C.c_int32), ("v_unit", C.c_int32), ("yarn_factor", C.c_float), ("yarn_fast", C.c_float), ("yarn_slow", C.c_float), ("yarn_original", C.c_int32)] +
                 [("ff_up_bias", C.c_void_p), ("ff_down_bias", C.c_void_p)] +
-                [(n, C.c_int32) for n in ("moe_identity", "moe_softmax", "moe_groups", "moe_keep", "moe_weight_output")] + [("moe_correction", C.c_void_p)])
+                [(n, C.c_int32) for n in ("moe_identity", "moe_softmax", "moe_groups", "moe_keep", "moe_weight_output")] + [("moe_correction", C.c_void_p)] +
+                [("moe_scale", C.c_float), ("out_bias", C.c_void_p), ("dist_slope", C.c_void_p)] + [(n, C.c_int32) for n in ("keep_first", "kv_from", "norm_parts")] +
+                [("conv_bias", C.c_void_p), ("skip", C.c_void_p)])
 
 
 class SeqDesc(C.Structure):
@@ -110,7 +112,8 @@ class SeqDesc(C.Structure):
     _fields_ = ([(n, C.c_int32) for n in ("n_layers", "width", "vocab", "canon_taps", "max_batch", "n_slots", "compute")] +
                 [("norm_eps", C.c_float), ("norm_offset", C.c_float), ("logit_scale", C.c_float)] +
                 [("embed", C.c_void_p), ("head", C.c_void_p), ("final_norm", C.c_void_p), ("layers", C.POINTER(SeqLayer))] +
-                [("embed_scale", C.c_float)] + [(n, C.c_int32) for n in ("loop_start", "loop_stop", "loop_times", "max_context", "norm_groups", "norm_center")])
+                [("embed_scale", C.c_float)] + [(n, C.c_int32) for n in ("loop_start", "loop_stop", "loop_times", "max_context", "norm_groups", "norm_center")] +
+                [("bigram", C.c_void_p)] + [(n, C.c_int64) for n in ("bigram_buckets", "bigram_mul_prev", "bigram_mul_cur")] + [("logit_softcap", C.c_float)])
 
 
 _LIB = None

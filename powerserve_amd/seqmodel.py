@@ -36,6 +36,14 @@ Mixers:
 Feed-forward: relu-gated dense with biases, or a mixture of squared-relu experts -- soft-max router in fp32 over experts AND identity experts (output = input), a
 correction added to the scores for the choice only, the choice limited to the best groups of neighbouring router rows, the chosen scores (not renormalised) on the
 experts' outputs, plus a shared expert for every token.
+
+Pupidra: POST-NORM layers,  x += ls1 * n1(mix(x)); x += ls2 * n2(mlp(x)): the sublayers read the residual stream itself, RMS norms with plain weights and a layer
+scale on what they put out (loaded as one vector, weight times scale).  A hashed bigram table is added to the embedding, the logits pass a soft cap.  Mixers:
+  mamba2            state-space recurrence with a scalar decay per head; x | B | C behind a short convolution with a bias; the gate before a norm in equal parts
+  attention         grouped-query attention over a sliding window and the first tokens of the sequence, a penalty slope_h * distance on the scores, unit-rms q and k per
+                    head, biases on all four projections; with 'kv_from' a layer reads another one's cached keys and values
+  latent_attention  as Pokatar's, with rotary on neighbouring pairs and plain frequencies
+Feed-forward: squared-relu experts behind a soft-max router in fp32, the chosen scores (not renormalised) times router.scale on the outputs, a shared expert.
 """
 from __future__ import annotations
 
@@ -48,9 +56,9 @@ import numpy as np
 from . import hip
 from .safetensors_io import SafeTensors
 
-MIX_WKV, MIX_DELTA, MIX_LATENT, MIX_WINATTN, MIX_GLA, MIX_MINGRU = 1, 2, 3, 4, 5, 6
+MIX_WKV, MIX_DELTA, MIX_LATENT, MIX_WINATTN, MIX_GLA, MIX_MINGRU, MIX_SSD = 1, 2, 3, 4, 5, 6, 7
 FF_NONE, FF_DENSE_XIELU, FF_DENSE_SWIGLU, FF_MOE_SWIGLU, FF_DENSE_RELU_GLU, FF_MOE_RELU2 = 0, 1, 2, 3, 4, 5
-LAYER_SEQUENTIAL, LAYER_PARALLEL, LAYER_PRENORM = 0, 1, 2
+LAYER_SEQUENTIAL, LAYER_PARALLEL, LAYER_PRENORM, LAYER_POSTNORM = 0, 1, 2, 3
 ROT_HALVES, ROT_NEIGHBOURS = 0, 1
 
 
@@ -278,10 +286,10 @@ def sink_attention_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str):
     L.out = up.mat(st.bf16_bits(m + "o"))
 
 
-def shared_key_latent_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str):
+def shared_key_latent_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str, pairing: int = ROT_HALVES):
     """Fill descriptor L with latent attention whose queries come straight from the input (MIX_LATENT with q_rank 0): q | dkv | g stacked, uk | uv stacked,
     causal (window 0) unless the configuration has a mask, frequency scaling from rot.scaling, a gate row per head where the file has one."""
-    L.kind, L.q_rank = MIX_LATENT, 0
+    L.kind, L.q_rank, L.rot_pairing = MIX_LATENT, 0, pairing
     L.heads, L.dim, L.vdim = int(mc["heads"]), int(mc["dim"]), int(mc.get("vdim") or mc["dim"])
     L.kv_rank, L.rot_dim = int(mc["kv_rank"]), int(mc["rot_dim"])
     rot = mc.get("rot") or {}
@@ -320,6 +328,7 @@ def relu_feed_forward(L, st: SafeTensors, up, p: str, mlp: dict, width: int, whe
         r = mlp["router"]
         L.ff_kind, L.ff, L.experts, L.top = FF_MOE_RELU2, int(mlp["expert"]["ff"]), int(r["experts"]), int(r["top"])
         L.moe_identity, L.moe_softmax, L.moe_weight_output = int(r.get("identity") or 0), 1, 1
+        L.moe_scale = float(r["scale"]) if r.get("scale") is not None else 1.0
         rows = L.experts + L.moe_identity
         gr = r.get("groups") or {}
         L.moe_groups, L.moe_keep = int(gr.get("count") or 0), int(gr.get("keep") or 0)
@@ -366,6 +375,101 @@ def _pokatar_layers(cfg: dict, st: SafeTensors, up) -> tuple[list, dict]:
     return layers, top
 
 
+def kept_window_attention_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str, layers: list):
+    """Fill descriptor L with grouped-query attention over a sliding window (mask.size) and the first tokens of the sequence (mask.keep_first), a distance penalty of
+    2^(-8 (h + 1) / heads) per head, q and k divided by their root mean square per head (no weight), biases where the file has them: MIX_WINATTN with those switches
+    on.  With 'kv_from' (the index of an earlier layer; `layers` holds their configurations) only queries are projected and that layer's cached rows are read."""
+    L.kind = MIX_WINATTN
+    L.heads, L.dim = int(mc["heads"]), int(mc["dim"])
+    L.kv_heads, L.vdim = int(mc.get("kv_heads") or L.heads), int(mc.get("vdim") or L.dim)
+    if L.heads % L.kv_heads:
+        raise ConfigError(f"{where}: {L.heads} heads over {L.kv_heads} key / value heads")
+    mask, source = mc.get("mask") or {}, mc.get("kv_from")
+    L.window, L.keep_first = int(mask.get("size") or 0), int(mask.get("keep_first") or 0)
+    L.rot_base, L.rot_pairing = 10000.0, ROT_NEIGHBOURS
+    L.scale = float(mc["scale"]) if mc.get("scale") is not None else L.dim ** -0.5
+    L.head_norm = 1
+    L.qnorm = up.vec(np.ones(L.dim, np.float32))
+    L.dist_slope = up.vec(np.exp2(-8.0 * (np.arange(L.heads) + 1.0) / L.heads))
+    names = ["q"]
+    if source is None:
+        L.knorm = up.vec(np.ones(L.dim, np.float32))
+        names += ["k", "v"]
+    else:
+        of = layers[source]["mixer"] if 0 <= source < len(layers) and layers[source]["type"] == "attention" else None
+        if of is None or of.get("kv_from") is not None:
+            raise ConfigError(f"{where}: kv_from {source} names no earlier attention layer with keys of its own")
+        for n, d in (("kv_heads", of["heads"]), ("dim", None), ("vdim", of["dim"])):
+            if int(of.get(n) or d) != getattr(L, n):
+                raise ConfigError(f"{where}: {n} {getattr(L, n)}, layer {source} has {int(of.get(n) or d)}")
+        L.kv_from = source + 1
+    size = {"q": L.heads * L.dim, "k": L.kv_heads * L.dim, "v": L.kv_heads * L.vdim}
+    for n in names:
+        if st.shape(m + n)[0] != size[n]:
+            raise ConfigError(f"tensor {m + n}: {st.shape(m + n)[0]} rows, the configuration gives {size[n]}")
+    L.in_cat = up.mat(_stack(st, [m + n for n in names]))
+    if any(m + n + ".b" in st for n in names):
+        L.in_bias = up.vec(np.concatenate([_expect(st, m + n + ".b", (size[n],)) if m + n + ".b" in st else np.zeros(size[n], np.float32) for n in names]))
+    L.out = up.mat(st.bf16_bits(m + "o"))
+    if m + "o.b" in st:
+        L.out_bias = up.vec(_expect(st, m + "o.b", (st.shape(m + "o")[0],)))
+
+
+def state_space_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str):
+    """Fill descriptor L with a state-space recurrence (MIX_SSD): z | x | B | C | dt is one projection, x | B | C pass a short convolution with a bias."""
+    L.kind = MIX_SSD
+    L.heads, L.vdim, L.dim, L.kv_heads = int(mc["heads"]), int(mc["vdim"]), int(mc["state"]), int(mc.get("groups") or 1)
+    L.conv_taps, L.norm_parts = int(mc["conv"]), int(mc.get("norm_groups") or 1)
+    inner, chan = L.heads * L.vdim, L.heads * L.vdim + 2 * L.kv_heads * L.dim
+    if L.heads % L.kv_heads or inner % L.norm_parts:
+        raise ConfigError(f"{where}: {L.heads} heads in {L.kv_heads} groups, {inner} numbers normed in {L.norm_parts} parts")
+    if st.shape(m + "in")[0] != inner + chan + L.heads:
+        raise ConfigError(f"tensor {m}in: {st.shape(m + 'in')[0]} rows, the configuration gives {inner + chan + L.heads}")
+    L.in_cat, L.out = up.mat(st.bf16_bits(m + "in")), up.mat(st.bf16_bits(m + "o"))
+    L.conv = up.vec(_expect(st, m + "conv", (chan, L.conv_taps)))
+    L.conv_bias = up.vec(_expect(st, m + "conv.b", (chan,)) if m + "conv.b" in st else np.zeros(chan, np.float32))
+    L.a_log, L.dt_bias, L.skip = (up.vec(_expect(st, m + n, (L.heads,))) for n in ("A_log", "dt_bias", "D"))
+    L.onorm = up.vec(_expect(st, m + "norm", (inner,)))
+
+
+def _pupidra_layers(cfg: dict, st: SafeTensors, up) -> tuple[list, dict]:
+    width = int(cfg["width"])
+    layers = []
+
+    def output_norm(p, n):  # RMS norm weight times layer scale: both multiply the normed output element by element
+        w = _expect(st, p + "norm" + n, (width,))
+        return up.vec(w * _expect(st, p + "ls" + n, (width,)) if p + "ls" + n in st else w)
+
+    for i, lc in enumerate(cfg["layers"]):
+        p, mc, kind = f"l{i}.", lc["mixer"], lc["type"]
+        L = hip.SeqLayer()
+        L.form, L.mix_scale = LAYER_POSTNORM, 1.0
+        L.norm1b = output_norm(p, "1")
+        if kind == "mamba2":
+            state_space_mixer(L, st, up, p + "mix.", mc, f"layer {i}")
+        elif kind == "attention":
+            kept_window_attention_mixer(L, st, up, p + "mix.", mc, f"layer {i}", cfg["layers"][:i])
+        elif kind == "latent_attention":
+            shared_key_latent_mixer(L, st, up, p + "mix.", mc, f"layer {i}", ROT_NEIGHBOURS)
+        else:
+            raise ConfigError(f"layer {i}: mixer type {kind!r} is not known")
+        if lc.get("mlp"):
+            if lc["mlp"].get("kind") != "moe":
+                raise ConfigError(f"layer {i}: feed-forward kind {lc['mlp'].get('kind')!r} is not known")
+            L.norm2b = output_norm(p, "2")
+            relu_feed_forward(L, st, up, p + "mlp.", lc["mlp"], width, f"layer {i}")
+        layers.append(L)
+    top = dict(width=width, vocab=int(cfg["vocab"]), canon_taps=1, norm_eps=float(cfg["norm"]["eps"]), norm_offset=0.0, logit_scale=1.0,
+               logit_softcap=float(cfg.get("logit_softcap") or 0.0), embed=up.mat(st.bf16_bits("embed")), head=up.mat(st.bf16_bits("head")),
+               final_norm=up.vec(_expect(st, "final.norm", (width,))))
+    big = (cfg.get("embedding") or {}).get("bigram")
+    if big:
+        if st.shape("bigram") != (int(big["buckets"]) + 1, width):
+            raise ConfigError(f"tensor bigram: shape {st.shape('bigram')}, the configuration gives {(int(big['buckets']) + 1, width)}")
+        top.update(bigram=up.mat(st.bf16_bits("bigram")), bigram_buckets=int(big["buckets"]), bigram_mul_prev=int(big["mul_prev"]), bigram_mul_cur=int(big["mul_cur"]))
+    return layers, top
+
+
 def _vobisun_layers(cfg: dict, st: SafeTensors, up) -> tuple[list, dict]:
     width = int(cfg["width"])
     taps = int((cfg.get("canon") or {}).get("taps") or 1)
@@ -405,7 +509,7 @@ def _vobisun_layers(cfg: dict, st: SafeTensors, up) -> tuple[list, dict]:
     return layers, top
 
 
-ARCHITECTURES = {"Ranutar": _ranutar_layers, "Vobisun": _vobisun_layers, "Zusolix": _zusolix_layers, "Pokatar": _pokatar_layers}
+ARCHITECTURES = {"Ranutar": _ranutar_layers, "Vobisun": _vobisun_layers, "Zusolix": _zusolix_layers, "Pokatar": _pokatar_layers, "Pupidra": _pupidra_layers}
 
 
 def read_config(model_dir: str) -> dict:

@@ -577,3 +577,165 @@ def run_pokatar(cfg, W, tokens, per_layer=None, attn_kw=None, latent_kw=None, mo
         if per_layer is not None:
             per_layer.append(x.copy())
     return centred_norm(x, W["final.norm"], eps) @ W["embed"].T
+
+
+# ------------------------------------------------------------------------------------------------ Pupidra
+# Post-norm layers,  x += ls1 * rms(mixer(x)) w;  x += ls2 * rms(ff(x)) w:  the sublayers read the residual stream itself.  The embedding has a second table
+# indexed by a hash of the previous and the present token.  Mixers: a state-space recurrence with a scalar decay per head (Mamba-2), attention with a
+# sliding window plus the first tokens of the sequence, a penalty per head that grows with the distance, unit-rms queries and keys and biases on every
+# projection -- possibly on another layer's keys and values --, and latent attention with neighbour-pair rotary and a gate per head.  The feed-forward is a
+# mixture of squared-relu experts whose soft-max scores are taken times a constant.  The logits pass a soft cap.
+
+
+def bigram_rows(tokens, bigram, use_previous=True):
+    """(previous * mul_prev + present * mul_cur) mod buckets, row `buckets` for a sequence's first token.  use_previous False: a WRONG model in which every
+    token counts as a first one."""
+    n = bigram["buckets"]
+    return [n if t == 0 or not use_previous else (int(tokens[t - 1]) * bigram["mul_prev"] + int(tokens[t]) * bigram["mul_cur"]) % n for t in range(len(tokens))]
+
+
+def state_space_scan(x, B, C, dt, a_log, D, carry=True, lose_at=None):
+    """S <- exp(-exp(a_log) dt) S + dt B x^T, y = S^T C + D x, head by head.  x [T, H, P], B / C [T, groups, N], dt [T, H] (after the softplus).
+    carry False: a WRONG model whose state is lost at every token; lose_at: ... in front of that token only."""
+    T, H, P = x.shape
+    G, N = B.shape[1:]
+    y = np.zeros((T, H, P))
+    for hd in range(H):
+        g = hd // (H // G)
+        S = np.zeros((N, P))
+        for t in range(T):
+            if not carry or t == lose_at:
+                S = np.zeros((N, P))
+            S = np.exp(-np.exp(a_log[hd]) * dt[t, hd]) * S + dt[t, hd] * np.outer(B[t, g], x[t, hd])
+            y[t, hd] = S.T @ C[t, g] + D[hd] * x[t, hd]
+    return y
+
+
+def gated_part_norm(y, z, w, parts, eps, gate_first=True):
+    """y * silu(z), then each of `parts` equal stretches divided by its own root mean square, times w.  gate_first False: a WRONG order (norm, then gate)."""
+    a = y * silu(z) if gate_first else y
+    T, n = a.shape
+    a = unit_rms(a.reshape(T, parts, n // parts), eps).reshape(T, n) * w
+    return a if gate_first else a * silu(z)
+
+
+def state_space_mixer(W, pre, h, mc, eps, carry=True, lose_at=None, use_D=True, use_filter=True, gate_first=True, one_group=False):
+    T = h.shape[0]
+    H, P, N, G = mc["heads"], mc["vdim"], mc["state"], mc["groups"]
+    inner = H * P
+    u = h @ W[pre + "in"].T
+    z, xbc, dt = u[:, :inner], u[:, inner:2 * inner + 2 * G * N], u[:, 2 * inner + 2 * G * N:]
+    assert dt.shape[1] == H and W[pre + "conv"].shape[1] == mc["conv"]
+    xbc = silu((time_conv(xbc, W[pre + "conv"]) if use_filter else xbc) + W[pre + "conv.b"])
+    x, B, C = xbc[:, :inner].reshape(T, H, P), xbc[:, inner:inner + G * N].reshape(T, G, N), xbc[:, inner + G * N:].reshape(T, G, N)
+    if one_group:  # a WRONG model in which every head reads the first group's B and C
+        B, C = np.repeat(B[:, :1], G, axis=1), np.repeat(C[:, :1], G, axis=1)
+    dt = softplus(dt + W[pre + "dt_bias"])
+    y = state_space_scan(x, B, C, dt, W[pre + "A_log"], W[pre + "D"] if use_D else np.zeros(H), carry, lose_at)
+    return gated_part_norm(y.reshape(T, inner), z, W[pre + "norm"], mc["norm_groups"], eps, gate_first) @ W[pre + "o"].T
+
+
+def kept_window_mask(T, size, keep):
+    """[i, j]: j <= i and (i - j < size or j < keep); size None: everything before the token."""
+    i, j = np.arange(T)[:, None], np.arange(T)[None, :]
+    return (j <= i) & ((i - j < (T if size is None else size)) | (j < keep))
+
+
+def distance_slopes(H):
+    return 2.0 ** (-8.0 * (np.arange(H) + 1.0) / H)
+
+
+def kept_window_attention(W, pre, h, mc, eps, source=None, size=None, keep=None, use_slopes=True, use_unit=True, use_bias=True):
+    """-> (output, (keys, values)).  source: the keys and values of another layer, read instead of own ones.  size / keep: WRONG masks."""
+    T = h.shape[0]
+    H, G, d, dv = mc["heads"], mc["kv_heads"], mc["dim"], mc["vdim"]
+    mask = mc.get("mask") or {}
+    size = mask.get("size") if size is None else size
+    keep = mask.get("keep_first", 0) if keep is None else keep
+
+    def proj(n):
+        return h @ W[pre + n].T + (W[pre + n + ".b"] if use_bias else 0.0)
+
+    unit = (lambda a: unit_rms(a, eps)) if use_unit else (lambda a: a)
+    q = unit(proj("q").reshape(T, H, d))
+    k, v = source if source is not None else (unit(proj("k").reshape(T, G, d)), proj("v").reshape(T, G, dv))
+    visible = kept_window_mask(T, size, keep)
+    distance = np.arange(T)[:, None] - np.arange(T)[None, :]
+    out = np.zeros((T, H, dv))
+    for hd in range(H):
+        g = hd // (H // G)
+        s = q[:, hd] @ k[:, g].T * mc["scale"] - (distance_slopes(H)[hd] * distance if use_slopes else 0.0)
+        s = np.where(visible, s, -np.inf)
+        e = np.exp(s - s.max(axis=1, keepdims=True))
+        out[:, hd] = e / e.sum(axis=1, keepdims=True) @ v[:, g]
+    return out.reshape(T, H * dv) @ W[pre + "o"].T + (W[pre + "o.b"] if use_bias else 0.0), (k, v)
+
+
+def neighbour_latent_attention(W, pre, h, mc, eps, reach=None, use_rotation=True, use_gate=True, use_latent_norm=True):
+    """Direct queries [dim plain | rot_dim rotated] per head, one normed latent and one rotated key part per token, neighbour-pair rotary, a gate per head."""
+    T = h.shape[0]
+    H, d, dr, dv, R = mc["heads"], mc["dim"], mc["rot_dim"], mc["vdim"], mc["kv_rank"]
+    base, dims = mc["rot"]["base"], mc["rot"]["dims"] if use_rotation else 0
+    q = (h @ W[pre + "q"].T).reshape(T, H, d + dr)
+    down = h @ W[pre + "dkv"].T
+    c = (unit_rms(down[:, :R], eps) if use_latent_norm else down[:, :R]) * W[pre + "dkv.norm"]
+    kr = np.stack([rotate_pairs(down[t, R:], t, base, dims) for t in range(T)])
+    qr = np.stack([rotate_pairs(q[t, :, d:], t, base, dims) for t in range(T)])
+    kp, v = (c @ W[pre + "uk"].T).reshape(T, H, d), (c @ W[pre + "uv"].T).reshape(T, H, dv)
+    gate = sigmoid(h @ W[pre + "g"].T) if use_gate else np.ones((T, H))
+    visible = kept_window_mask(T, reach, 0)
+    out = np.zeros((T, H, dv))
+    for hd in range(H):
+        s = np.where(visible, (q[:, hd, :d] @ kp[:, hd].T + qr[:, hd] @ kr.T) * mc["scale"], -np.inf)
+        e = np.exp(s - s.max(axis=1, keepdims=True))
+        out[:, hd] = e / e.sum(axis=1, keepdims=True) @ v[:, hd] * gate[:, hd:hd + 1]
+    return out.reshape(T, H * dv) @ W[pre + "o"].T
+
+
+def scaled_experts(W, pre, h, mlp, use_scale=True, use_shared=True, renormalise=False):
+    """Soft-max over all experts, the `top` largest as they are, times router.scale, on the experts' outputs.  renormalise: a WRONG model."""
+    r = mlp["router"]
+    out = np.zeros_like(h)
+    for t in range(h.shape[0]):
+        z = W[pre + "router"] @ h[t]
+        s = np.exp(z - z.max())
+        s /= s.sum()
+        chosen = np.argsort(-s, kind="stable")[:r["top"]]
+        for e in chosen:
+            w = s[e] / (s[chosen].sum() if renormalise else 1.0) * (r["scale"] if use_scale else 1.0)
+            out[t] += w * squared_relu_expert(W, f"{pre}e{e}.", h[t])
+    if mlp.get("shared") and use_shared:
+        out += squared_relu_expert(W, pre + "shared.", h)
+    return out
+
+
+def run_pupidra(cfg, W, tokens, per_layer=None, use_bigram=True, use_previous=True, use_layer_scale=True, use_cap=True, share=True, attn_kw=None, latent_kw=None, ssm_kw=None, moe_kw=None):
+    """-> logits [T, vocab]; per_layer (a list) receives the residual stream after every layer.  share False: a WRONG model in which a layer with kv_from uses
+    the keys and values of the latest attention layer before it that has its own instead of the named one's."""
+    W = {k: np.asarray(v, dtype=np.float64) for k, v in W.items()}
+    eps = cfg["norm"]["eps"]
+    x = W["embed"][np.asarray(tokens)]
+    if use_bigram and (cfg.get("embedding") or {}).get("bigram"):
+        x = x + W["bigram"][bigram_rows(tokens, cfg["embedding"]["bigram"], use_previous)]
+    cached, latest = {}, None
+    for i, lc in enumerate(cfg["layers"]):
+        p, mc, kind = f"l{i}.", lc["mixer"], lc["type"]
+        if kind == "mamba2":
+            y = state_space_mixer(W, p + "mix.", x, mc, eps, **(ssm_kw or {}))
+        elif kind == "attention":
+            j = mc.get("kv_from")
+            y, cached[i] = kept_window_attention(W, p + "mix.", x, mc, eps, None if j is None else cached[j if share else latest], **(attn_kw or {}))
+            latest = i if j is None else latest
+        elif kind == "latent_attention":
+            y = neighbour_latent_attention(W, p + "mix.", x, mc, eps, **(latent_kw or {}))
+        else:
+            raise ValueError(kind)
+        x = x + plain_norm(y, W[p + "norm1"], eps) * (W[p + "ls1"] if use_layer_scale else 1.0)
+        if lc.get("mlp"):
+            y = scaled_experts(W, p + "mlp.", x, lc["mlp"], **(moe_kw or {}))
+            x = x + plain_norm(y, W[p + "norm2"], eps) * (W[p + "ls2"] if use_layer_scale else 1.0)
+        if per_layer is not None:
+            per_layer.append(x.copy())
+    logits = plain_norm(x, W["final.norm"], eps) @ W["head"].T
+    cap = cfg.get("logit_softcap")
+    return cap * np.tanh(logits / cap) if cap and use_cap else logits
