@@ -36,11 +36,27 @@ SIZES = {
                     order="aalaal", layers=6, beside="z2048x6"),
     "p4096x3": dict(design="Pokatar", width=4096, ff=14336, heads=32, kv_heads=8, dim=128, kv_rank=512, rot_dim=64, experts=8, identity=2, groups=(5, 3), top=2,
                     order="ala", layers=3, beside="z4096x3"),
+    # Pupidra (post-norm layers; m = state-space recurrence with inner size 2 x width in heads of 64, state 128, 8 groups, a = attention over a window and the first
+    # tokens, s = the same on the keys and values of the a layer before it, l = latent attention with neighbour-pair rotary; every feed-forward 8 squared-relu
+    # experts, top 2, plus a shared expert, of the Pokatar sizes) beside the Pokatar model of equal width, feed-forward sizes, head counts and layers
+    "u2048x6": dict(design="Pupidra", width=2048, ff=8192, heads=16, kv_heads=4, dim=128, window=1024, keep_first=64, kv_rank=512, rot_dim=64, state=128, groups=8, experts=8,
+                    top=2, order="mmalsl", layers=6, beside="p2048x6"),
+    "u4096x3": dict(design="Pupidra", width=4096, ff=14336, heads=32, kv_heads=8, dim=128, window=1024, keep_first=64, kv_rank=512, rot_dim=64, state=128, groups=8, experts=8,
+                    top=2, order="mal", layers=3, beside="p4096x3"),
 }
 
 
 def config(z: dict, vocab: int = 4096) -> dict:
     H, d = z["heads"], z["dim"]
+    if z.get("design") == "Pupidra":
+        kinds = {"m": ("mamba2", synth.pupidra_mamba2(2 * z["width"] // 64, 64, z["state"], z["groups"], 4, z["groups"])),
+                 "l": ("latent_attention", synth.pupidra_latent(H, d, z["rot_dim"], d, z["kv_rank"], float((d + z["rot_dim"]) ** -0.5), 5e5))}
+        layers = []
+        for i, k in enumerate(z["order"]):
+            own = max([j for j in range(i) if z["order"][j] == "a"], default=None)
+            mixer = kinds.get(k) or ("attention", synth.pupidra_attention(H, z["kv_heads"], d, d, 1.0, z["window"], z["keep_first"], own if k == "s" else None))
+            layers.append(synth.pupidra_layer(*mixer, moe=(z["experts"], z["top"], z["ff"] * 3 // 8, 2.0), shared=z["ff"] * 3 // 4))
+        return synth.pupidra_config(z["width"], vocab, layers, bigram=(4093, 31, 17), softcap=30.0)
     if z.get("design") == "Pokatar":
         att = synth.pokatar_attention(H, z["kv_heads"], d, d, float(d ** -0.5))
         lat = synth.pokatar_latent(H, d, z["rot_dim"], d, z["kv_rank"], float((d + z["rot_dim"]) ** -0.5), 5e5, (8.0, 4096, 16.0, 2.0))
@@ -114,10 +130,11 @@ def run_size(ctx, name: str, prompt_len: int, steps: int, max_batch: int, seed: 
     out["decode_hbm_frac"] = m.weight_bytes_per_token * steps / dec / 1e9 / HBM_PEAK_GBS
     flops_tok = 2.0 * (m.weight_bytes_per_token / 2 - cfg["vocab"] * cfg["width"])
     out["prefill_mfma_frac"] = flops_tok * (prompt_len - 1) / pre / 1e12 / MFMA_BF16_PEAK_TFLOPS
-    us, by, fl = _kernel(ctx, m, 0, 1, 20)
-    out["ff_up_matvec"] = {"us": us, "GBs": by / us / 1e3, "hbm_frac": by / us / 1e3 / HBM_PEAK_GBS}
-    us, by, fl = _kernel(ctx, m, 0, max_batch, 5)
-    out["ff_up_matmul"] = {"tokens": max_batch, "us": us, "TFLOPs": fl / us / 1e6, "mfma_frac": fl / us / 1e6 / MFMA_BF16_PEAK_TFLOPS}
+    if any((lc.get("mlp") or {}).get("kind") == "dense" for lc in cfg["layers"]):
+        us, by, fl = _kernel(ctx, m, 0, 1, 20)
+        out["ff_up_matvec"] = {"us": us, "GBs": by / us / 1e3, "hbm_frac": by / us / 1e3 / HBM_PEAK_GBS}
+        us, by, fl = _kernel(ctx, m, 0, max_batch, 5)
+        out["ff_up_matmul"] = {"tokens": max_batch, "us": us, "TFLOPs": fl / us / 1e6, "mfma_frac": fl / us / 1e6 / MFMA_BF16_PEAK_TFLOPS}
     if z.get("experts"):  # the experts' grouped products: up (gate / up rows, SiLU pair) and down, a single token and a portion
         for which, key in ((2, "moe_up"), (3, "moe_down")):
             us, by, fl = _kernel(ctx, m, which, 1, 20)

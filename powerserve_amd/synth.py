@@ -434,11 +434,101 @@ def _pokatar_tensors(cfg: dict, seed: int) -> dict:
     return t
 
 
+def pupidra_mamba2(heads: int, vdim: int, state: int, groups: int, conv: int, norm_groups: int) -> dict:
+    """mixer entry of a Pupidra state-space layer"""
+    return {"heads": int(heads), "vdim": int(vdim), "state": int(state), "groups": int(groups), "conv": int(conv), "norm_groups": int(norm_groups)}
+
+
+def pupidra_attention(heads: int, kv_heads: int, dim: int, vdim: int, scale: float, size: int, keep_first: int, kv_from: int | None = None) -> dict:
+    """mixer entry of a Pupidra attention layer; kv_from: the index of the layer whose keys and values it reads"""
+    mc = {"heads": int(heads), "kv_heads": int(kv_heads), "dim": int(dim), "vdim": int(vdim), "scale": float(scale), "mask": {"size": int(size), "keep_first": int(keep_first)}}
+    if kv_from is not None:
+        mc["kv_from"] = int(kv_from)
+    return mc
+
+
+def pupidra_latent(heads: int, dim: int, rot_dim: int, vdim: int, kv_rank: int, scale: float, base: float = 10000.0) -> dict:
+    """mixer entry of a Pupidra latent-attention layer"""
+    return pokatar_latent(heads, dim, rot_dim, vdim, kv_rank, scale, base)
+
+
+def pupidra_layer(kind: str, mixer: dict, moe: tuple | None = None, shared: int | None = None) -> dict:
+    """One entry of a Pupidra configuration's 'layers'.  kind 'mamba2' / 'attention' / 'latent_attention'; moe = (experts, top, expert ff, scale) or None (no
+    feed-forward); shared = the shared expert's ff or None."""
+    mlp = None
+    if moe:
+        experts, top, eff, scale = moe
+        mlp = {"kind": "moe", "router": {"experts": int(experts), "top": int(top), "scale": float(scale)}, "expert": {"ff": int(eff)}}
+        if shared:
+            mlp["shared"] = {"ff": int(shared)}
+    return {"type": kind, "mixer": dict(mixer), "mlp": mlp}
+
+
+def pupidra_config(width: int, vocab: int, layers: list, bigram: tuple | None = None, softcap: float | None = None, eps: float = 1e-6) -> dict:
+    """bigram: (buckets, mul_prev, mul_cur) or None"""
+    cfg = {"architecture": "Pupidra", "layers": layers, "norm": {"eps": float(eps)}, "vocab": int(vocab), "width": int(width)}
+    if bigram:
+        cfg["embedding"] = {"bigram": dict(zip(("buckets", "mul_prev", "mul_cur"), map(int, bigram)))}
+    if softcap:
+        cfg["logit_softcap"] = float(softcap)
+    return cfg
+
+
+def _pupidra_tensors(cfg: dict, seed: int) -> dict:
+    rng = np.random.default_rng(seed)
+    W = cfg["width"]
+
+    def lin(n, k, gain=1.0):
+        return rng.standard_normal((n, k), dtype=np.float32) * np.float32(gain / np.sqrt(k))
+
+    def vec(n, std=0.1, mean=0.0):
+        return (rng.standard_normal(n, dtype=np.float32) * np.float32(std) + np.float32(mean)).astype(np.float32)
+
+    t = {"embed": rng.standard_normal((cfg["vocab"], W), dtype=np.float32)}
+    if (cfg.get("embedding") or {}).get("bigram"):
+        t["bigram"] = rng.standard_normal((cfg["embedding"]["bigram"]["buckets"] + 1, W), dtype=np.float32)
+    for i, lc in enumerate(cfg["layers"]):
+        p, m, mc = f"l{i}.", f"l{i}.mix.", lc["mixer"]
+        t[p + "norm1"], t[p + "ls1"] = vec(W, 0.2, 1.0), vec(W, 0.3, 0.8)
+        H, dv = mc["heads"], mc["vdim"]
+        if lc["type"] == "mamba2":
+            inner, chan = H * dv, H * dv + 2 * mc["groups"] * mc["state"]
+            t[m + "in"], t[m + "conv"], t[m + "conv.b"] = lin(inner + chan + H, W), vec(chan * mc["conv"], 0.6).reshape(chan, mc["conv"]), vec(chan, 0.3)
+            t[m + "dt_bias"], t[m + "A_log"] = vec(H, 0.7, -1.5), np.log(rng.uniform(0.3, 3.0, H)).astype(np.float32)
+            t[m + "D"], t[m + "norm"] = vec(H, 0.5, 1.0), vec(inner, 0.2, 1.0)
+        elif lc["type"] == "attention":
+            d, G = mc["dim"], mc["kv_heads"]
+            rows = {"q": H * d} if mc.get("kv_from") is not None else {"q": H * d, "k": G * d, "v": G * dv}
+            for n, r in rows.items():
+                t[m + n], t[m + n + ".b"] = lin(r, W), vec(r, 0.3)
+            t[m + "o.b"] = vec(W, 0.3)
+        elif lc["type"] == "latent_attention":
+            d, R, dr = mc["dim"], mc["kv_rank"], mc["rot_dim"]
+            t[m + "q"], t[m + "dkv"], t[m + "dkv.norm"] = lin(H * (d + dr), W, 1.5), lin(R + dr, W, 1.5), vec(R, 0.3, 1.0)
+            t[m + "uk"], t[m + "uv"], t[m + "g"] = lin(H * d, R, 1.5), lin(H * dv, R), lin(H, W, 2.0)
+        else:
+            raise ValueError(lc["type"])
+        t[m + "o"] = lin(W, H * dv)
+        mlp = lc.get("mlp")
+        if mlp:
+            t[p + "norm2"], t[p + "ls2"] = vec(W, 0.2, 1.0), vec(W, 0.3, 0.8)
+            q, r, ff = p + "mlp.", mlp["router"], mlp["expert"]["ff"]
+            for e in range(r["experts"]):
+                t[f"{q}e{e}.up"], t[f"{q}e{e}.down"] = lin(ff, W, 1.5), lin(W, ff)
+            t[q + "router"] = lin(r["experts"], W, 2.0)
+            if mlp.get("shared"):
+                t[q + "shared.up"], t[q + "shared.down"] = lin(mlp["shared"]["ff"], W, 1.5), lin(W, mlp["shared"]["ff"])
+    t["final.norm"], t["head"] = vec(W, 0.2, 1.0), lin(cfg["vocab"], W, 3.0)
+    return t
+
+
 def seq_tensors(cfg: dict, seed: int = 0, decay_rank: int = 8) -> dict:
     """Random-init tensors of a layer-list configuration, name -> float32 array already rounded to bfloat16 (what the file will hold)."""
     from .safetensors_io import f32_to_bf16_bits
-    if cfg.get("architecture") in ("Vobisun", "Zusolix", "Pokatar"):
-        t = {"Vobisun": lambda: _parallel_tensors(cfg, seed, decay_rank), "Zusolix": lambda: _zusolix_tensors(cfg, seed), "Pokatar": lambda: _pokatar_tensors(cfg, seed)}[cfg["architecture"]]()
+    makers = {"Vobisun": lambda: _parallel_tensors(cfg, seed, decay_rank), "Zusolix": lambda: _zusolix_tensors(cfg, seed), "Pokatar": lambda: _pokatar_tensors(cfg, seed),
+              "Pupidra": lambda: _pupidra_tensors(cfg, seed)}
+    if cfg.get("architecture") in makers:
+        t = makers[cfg["architecture"]]()
         return {k: (f32_to_bf16_bits(v).astype(np.uint32) << 16).view(np.float32).reshape(v.shape) for k, v in t.items()}
     rng = np.random.default_rng(seed)
     W, taps = cfg["width"], cfg["canon"]["taps"]

@@ -93,7 +93,10 @@ def test_ctypes_descriptors_match_the_header(tmp_path):
                    'printf("%zu %zu %zu %zu %zu %zu %zu\\n", offsetof(ps_seq_layer, res_scale), offsetof(ps_seq_layer, depth_mix), offsetof(ps_seq_layer, softcap), '
                    'offsetof(ps_seq_layer, qtemp_every), offsetof(ps_seq_layer, experts), offsetof(ps_seq_layer, shared_down), offsetof(ps_seq_desc, norm_groups));'
                    'printf("%zu %zu %zu %zu %zu %zu %zu\\n", offsetof(ps_seq_layer, head_norm), offsetof(ps_seq_layer, yarn_factor), offsetof(ps_seq_layer, yarn_original), '
-                   'offsetof(ps_seq_layer, ff_up_bias), offsetof(ps_seq_layer, moe_identity), offsetof(ps_seq_layer, moe_correction), offsetof(ps_seq_desc, norm_center));return 0;}\n')
+                   'offsetof(ps_seq_layer, ff_up_bias), offsetof(ps_seq_layer, moe_identity), offsetof(ps_seq_layer, moe_correction), offsetof(ps_seq_desc, norm_center));'
+                   'printf("%zu %zu %zu %zu %zu %zu %zu %zu %zu\\n", offsetof(ps_seq_layer, moe_scale), offsetof(ps_seq_layer, out_bias), offsetof(ps_seq_layer, dist_slope), '
+                   'offsetof(ps_seq_layer, keep_first), offsetof(ps_seq_layer, kv_from), offsetof(ps_seq_layer, norm_parts), offsetof(ps_seq_layer, skip), '
+                   'offsetof(ps_seq_desc, bigram), offsetof(ps_seq_desc, logit_softcap));return 0;}\n')
     exe = str(tmp_path / "sz")
     subprocess.run(["gcc", "-I" + os.path.join(ROOT, "include"), str(src), "-o", exe], check=True)
     got = [int(x) for x in subprocess.run([exe], check=True, capture_output=True, text=True).stdout.split()]
@@ -103,7 +106,9 @@ def test_ctypes_descriptors_match_the_header(tmp_path):
                    hip.SeqLayer.res_scale.offset, hip.SeqLayer.depth_mix.offset, hip.SeqLayer.softcap.offset, hip.SeqLayer.qtemp_every.offset, hip.SeqLayer.experts.offset,
                    hip.SeqLayer.shared_down.offset, hip.SeqDesc.norm_groups.offset,
                    hip.SeqLayer.head_norm.offset, hip.SeqLayer.yarn_factor.offset, hip.SeqLayer.yarn_original.offset, hip.SeqLayer.ff_up_bias.offset,
-                   hip.SeqLayer.moe_identity.offset, hip.SeqLayer.moe_correction.offset, hip.SeqDesc.norm_center.offset]
+                   hip.SeqLayer.moe_identity.offset, hip.SeqLayer.moe_correction.offset, hip.SeqDesc.norm_center.offset,
+                   hip.SeqLayer.moe_scale.offset, hip.SeqLayer.out_bias.offset, hip.SeqLayer.dist_slope.offset, hip.SeqLayer.keep_first.offset, hip.SeqLayer.kv_from.offset,
+                   hip.SeqLayer.norm_parts.offset, hip.SeqLayer.skip.offset, hip.SeqDesc.bigram.offset, hip.SeqDesc.logit_softcap.offset]
 
 
 def test_plain_statement_is_causal_and_windowed():
@@ -364,6 +369,87 @@ def test_plain_pokatar_statement_reach_and_pieces():
         sc = np.exp(z) / np.exp(z).sum()
         keep = np.argsort(-(sc + W["l0.mlp.correction"]))[:2]  # (five groups of one, two stay: the group limit changes nothing here)
         assert np.allclose(full[i], sum(sc[e] * (seq_oracle.squared_relu_expert(W, "l0.mlp.e%d." % e, h[i]) if e < 3 else h[i]) for e in keep))
+
+
+UCFG = synth.pupidra_config(24, 30, [
+    synth.pupidra_layer("mamba2", synth.pupidra_mamba2(6, 5, 7, 3, 4, 2), (3, 2, 8, 1.5), 5),
+    synth.pupidra_layer("attention", synth.pupidra_attention(4, 2, 6, 10, 0.25, 9, 3), (4, 1, 6, 2.0)),
+    synth.pupidra_layer("latent_attention", synth.pupidra_latent(3, 6, 4, 5, 7, 0.3, 77.0)),
+    synth.pupidra_layer("attention", synth.pupidra_attention(2, 2, 6, 10, 0.5, 5, 8, kv_from=1))], bigram=(11, 3, 2), softcap=20.0, eps=1e-5)
+
+
+def test_pupidra_configuration_maps_onto_layer_descriptors(tmp_path):
+    t = synth.write_seq_model_dir(str(tmp_path), UCFG, 1)
+    cfg = seqmodel.read_config(str(tmp_path))
+    up = FakeUp()
+    st = safetensors_io.SafeTensors(str(tmp_path / "model.safetensors"))
+    layers, top = seqmodel.ARCHITECTURES[cfg["architecture"]](cfg, st, up)
+    bits = safetensors_io.f32_to_bf16_bits
+    assert (top["width"], top["vocab"], top["norm_offset"], top["logit_softcap"], top["bigram_buckets"], top["bigram_mul_prev"], top["bigram_mul_cur"]) == (24, 30, 0.0, 20.0, 11, 3, 2)
+    assert up.mats[top["bigram"] - 1001].shape == (12, 24) and top["head"] != top["embed"]
+    m, a, b, c = layers
+    assert all(x.form == seqmodel.LAYER_POSTNORM and x.norm1 is None and x.norm2 is None and x.canon1 is None for x in layers)
+    # the layer scale is part of the output norm's weight
+    assert np.array_equal(up.vecs[m.norm1b - 1], t["l0.norm1"] * t["l0.ls1"]) and np.array_equal(up.vecs[m.norm2b - 1], t["l0.norm2"] * t["l0.ls2"]) and b.norm2b is None
+    # the recurrence: one stacked projection as the file has it
+    assert (m.kind, m.heads, m.vdim, m.dim, m.kv_heads, m.conv_taps, m.norm_parts) == (seqmodel.MIX_SSD, 6, 5, 7, 3, 4, 2)
+    assert up.mats[m.in_cat - 1001].shape == (30 + 30 + 21 + 21 + 6, 24) and up.vecs[m.conv - 1].shape == (72, 4) and up.vecs[m.conv_bias - 1].shape == (72,)
+    assert all(up.vecs[getattr(m, n) - 1].shape == (6,) for n in ("a_log", "dt_bias", "skip")) and up.vecs[m.onorm - 1].shape == (30,)
+    # attention: q | k | v stacked with their biases, a bias on the way out, unit weights for the norms, a slope per head
+    assert (a.kind, a.heads, a.kv_heads, a.dim, a.vdim, a.window, a.keep_first, a.pool, a.rot_dims, a.gated, a.head_norm, a.v_unit, a.kv_from) == (
+        seqmodel.MIX_WINATTN, 4, 2, 6, 10, 9, 3, 0, 0, 0, 1, 0, 0)
+    assert np.array_equal(up.mats[a.in_cat - 1001], np.concatenate([bits(t["l1.mix." + n]) for n in "qkv"])) and up.mats[a.in_cat - 1001].shape == (24 + 12 + 20, 24)
+    assert np.array_equal(up.vecs[a.in_bias - 1], np.concatenate([t["l1.mix." + n + ".b"] for n in "qkv"])) and np.array_equal(up.vecs[a.out_bias - 1], t["l1.mix.o.b"])
+    assert np.array_equal(up.vecs[a.dist_slope - 1], np.float32([2.0 ** -2, 2.0 ** -4, 2.0 ** -6, 2.0 ** -8])) and np.array_equal(up.vecs[a.qnorm - 1], np.ones(6)) and np.array_equal(up.vecs[a.knorm - 1], np.ones(6))
+    # a layer on another one's keys and values has queries only
+    assert (c.kv_from, c.heads, c.kv_heads, c.window, c.keep_first, c.knorm) == (2, 2, 2, 5, 8, None)
+    assert np.array_equal(up.mats[c.in_cat - 1001], bits(t["l3.mix.q"])) and np.array_equal(up.vecs[c.in_bias - 1], t["l3.mix.q.b"])
+    assert (b.kind, b.q_rank, b.kv_rank, b.rot_dim, b.rot_dims, b.rot_pairing, b.gated, b.window, b.yarn_factor) == (seqmodel.MIX_LATENT, 0, 7, 4, 4, seqmodel.ROT_NEIGHBOURS, 1, 0, 0.0)
+    assert (m.ff_kind, m.ff, m.experts, m.top, m.shared_ff, m.moe_softmax, m.moe_weight_output, m.moe_identity, m.moe_groups, m.moe_norm_top, m.moe_scale) == (
+        seqmodel.FF_MOE_RELU2, 8, 3, 2, 5, 1, 1, 0, 0, 0, 1.5)
+    assert b.ff_kind == c.ff_kind == seqmodel.FF_NONE and a.shared_up is None and a.moe_scale == 2.0
+    # what the file and the configuration do not have does not exist
+    less = {n: st.f32(n) for n in st.names() if not n.endswith(".b") and ".ls" not in n and n != "bigram"}
+    cfg2 = json.loads(json.dumps(UCFG))
+    del cfg2["embedding"], cfg2["logit_softcap"], cfg2["layers"][1]["mixer"]["mask"], cfg2["layers"][0]["mlp"]["router"]["scale"]
+    synth.write_seq_model_dir(str(tmp_path / "less"), cfg2, 1, tensors=less)
+    layers, top = seqmodel.ARCHITECTURES["Pupidra"](cfg2, safetensors_io.SafeTensors(str(tmp_path / "less" / "model.safetensors")), FakeUp())
+    m, a, b, c = layers
+    assert "bigram" not in top and top["logit_softcap"] == 0.0 and (a.window, a.keep_first, a.in_bias, a.out_bias, c.in_bias, m.moe_scale) == (0, 0, None, None, None, 1.0)
+    for i, key, val in ((1, "type", "conveyor"), (1, "mlp", {"kind": "dense", "ff": 8}), (3, "kv_from", 2), (3, "kv_from", 3), (3, "kv_from", 7), (3, "dim", 7), (3, "kv_heads", 1), (0, "groups", 4), (0, "norm_groups", 4)):
+        bad = json.loads(json.dumps(UCFG))
+        (bad["layers"][i] if key in ("type", "mlp") else bad["layers"][i]["mixer"])[key] = val
+        with pytest.raises(seqmodel.ConfigError):
+            seqmodel.ARCHITECTURES["Pupidra"](bad, st, FakeUp())
+
+
+def test_plain_pupidra_statement_reach_and_pieces():
+    """causal; the window with its kept first tokens by hand; the slopes of a head count that is no power of two; the bigram rows; the recurrence against its closed
+    form; the gate in front of the norm"""
+    t = synth.seq_tensors(UCFG, 2)
+    rng = np.random.default_rng(0)
+    a = rng.integers(0, 30, 20)
+    b = a.copy()
+    b[6] = (b[6] + 1) % 30
+    la, lb = seq_oracle.run_pupidra(UCFG, t, a), seq_oracle.run_pupidra(UCFG, t, b)
+    assert np.array_equal(la[:6], lb[:6]) and min(np.abs(la[i] - lb[i]).max() for i in range(6, 20)) > 1e-6 and np.abs(la).max() < 20.0
+    mask = seq_oracle.kept_window_mask(8, 3, 2)
+    assert [list(np.flatnonzero(r)) for r in mask] == [[0], [0, 1], [0, 1, 2], [0, 1, 2, 3], [0, 1, 2, 3, 4], [0, 1, 3, 4, 5], [0, 1, 4, 5, 6], [0, 1, 5, 6, 7]]
+    assert np.allclose(seq_oracle.distance_slopes(3), [2 ** (-8 / 3), 2 ** (-16 / 3), 2 ** -8.0])
+    assert seq_oracle.bigram_rows([4, 9, 0], {"buckets": 11, "mul_prev": 3, "mul_cur": 2}) == [11, (4 * 3 + 9 * 2) % 11, (9 * 3) % 11]
+    # S_t = sum_s prod_(s < r <= t) g_r dt_s B_s x_s^T
+    T, H, P, G, N = 9, 4, 3, 2, 5
+    x, B, C, dt = rng.standard_normal((T, H, P)), rng.standard_normal((T, G, N)), rng.standard_normal((T, G, N)), rng.random((T, H)) + 0.1
+    al, D = rng.standard_normal(H), rng.standard_normal(H)
+    y = seq_oracle.state_space_scan(x, B, C, dt, al, D)
+    for hd in range(H):
+        cum = np.cumsum(-np.exp(al[hd]) * dt[:, hd])
+        for i in range(T):
+            want = sum(np.exp(cum[i] - cum[j]) * dt[j, hd] * (C[i, hd // 2] @ B[j, hd // 2]) * x[j, hd] for j in range(i + 1)) + D[hd] * x[i, hd]
+            assert np.allclose(y[i, hd], want)
+    u, z = rng.standard_normal((2, 6)), rng.standard_normal((2, 6))
+    n = seq_oracle.gated_part_norm(u, z, np.ones(6), 3, 0.0)
+    assert np.allclose(np.mean(n.reshape(2, 3, 2) ** 2, axis=-1), 1.0) and np.allclose(n, seq_oracle.gated_part_norm(2.0 * u, z, np.ones(6), 3, 0.0))
 
 
 def test_the_small_library_exports_what_its_models_need():
