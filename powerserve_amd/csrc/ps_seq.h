@@ -122,6 +122,13 @@ void psk_gate_partnorm(hipStream_t st, float *o, int64_t ldo, const float *z, in
 // o[t][h][:] = o / sqrt(mean_j o^2 + eps) * w(h, :) * silu(g[t][h][:]);  w_stride = dv (a weight per head) or 0 (one shared by the heads)
 void psk_headnorm_gate(hipStream_t st, float *o, int64_t ldo, const float *g, int64_t ldg, const float *w, int w_stride, float eps, int H, int dv, int T);
 
+// ---- k_ssd.hip
+// psk_ssd_scan for a portion, in chunks of 64 tokens on the fp32 matrix cores (same arguments; the same result up to rounding); _ok: the sizes it takes.
+bool psk_ssd_chunked_ok(int N, int P);
+size_t psk_ssd_chunked_scratch(int H, int N, int P, int T);
+void psk_ssd_chunked(hipStream_t st, const ps_seq_step *step, int64_t state_off, const float *x, const float *B, const float *C, int64_t ld, const float *dtraw, int64_t ldb,
+                     const float *a_log, const float *dt_bias, const float *skip, int H, int G, int N, int P, int T, float *scratch, float *o, int64_t ldo);
+
 // ---- k_moe.hip
 // Router of a mixture of experts, fp32: scores = sigmoid(router h[t]), or (softmax) the soft-max over all `experts` rows; choice scores = scores + correction (NULL: none);
 // with n_groups > 0 only rows of the `keep` groups (equal runs of neighbours) with the largest best choice score stay in the race; the `top` largest choice scores

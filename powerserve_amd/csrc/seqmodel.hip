@@ -67,6 +67,7 @@ struct ps_hip_seq {
     int32_t *moe_sel = nullptr, *moe_seg = nullptr, *moe_list = nullptr; // mixture of experts: expert per slot, the slots sorted by expert
     float *moe_wgt = nullptr, *moe_sg = nullptr, *moe_y = nullptr;       // weight per slot, the shared expert's gate per token, per-slot results (top > 1)
     float *win_scratch = nullptr; // the windowed attention's single-token partials
+    float *ssd_scratch = nullptr; // the chunked state-space recurrence: a state per chunk
     float *abs_scratch = nullptr; // the absorbed single-token attention's folded queries, attended latents and per-tile partials
     void *pack = nullptr; // the wide mat-mul's bfloat16 operand copy
     size_t pack_bytes = 0;
@@ -98,6 +99,8 @@ __global__ void seq_advance_kernel(ps_seq_step *s, const int32_t *amax, int32_t 
     s->token0 = id;
     s->pos0 += 1;
 }
+
+static const int SSD_CHUNKED_FROM = 32; // tokens from which a portion's state-space recurrence runs in chunks (fewer: the scan)
 
 static int seq_fail(ps_hip_ctx *c, const std::string &msg) { c->err = msg; return 2; }
 
@@ -438,6 +441,11 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
                 wb = std::max(wb, psk_winattn_step_scratch(P.d.heads, P.d.vdim, P.d.window, psk_front_store{P.off_pool, P.d.pool, P.d.keep_first}, m->max_context));
         });
         if (wb) ok = ok && alloc((void **)&m->win_scratch, wb);
+        size_t sb = 0;
+        mixers([&](LayerPlan &P) {
+            if (P.d.kind == PS_MIX_SSD && B >= SSD_CHUNKED_FROM && psk_ssd_chunked_ok(P.d.dim, P.d.vdim)) sb = std::max(sb, psk_ssd_chunked_scratch(P.d.heads, P.d.dim, P.d.vdim, (int)B));
+        });
+        if (sb) ok = ok && alloc((void **)&m->ssd_scratch, sb);
     }
     if (desc->compute == 0) { // the wide mat-mul's operand copy: the widest input of any matrix x a portion's rows, or the window's rows x the latent
         int64_t kmax = W, kvrows = 0, kvk = 0;
@@ -603,8 +611,11 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
             const int64_t inner = H * dv, GN = (int64_t)l.kv_heads * d;
             if (!P.in_ld) psk_dense(st, mm(l.in_cat, in, W, t1, ld1));
             psk_causal_conv(st, m->step, P.off_conv, t1 + inner, ld1, l.conv, l.conv_taps, 1, P.cqkv, T, m->t2, P.cqkv, l.conv_bias);
-            psk_ssd_scan(st, m->step, P.off_S, m->t2, m->t2 + inner, m->t2 + inner + GN, P.cqkv, t1 + inner + P.cqkv, ld1, l.a_log, l.dt_bias, l.skip, (int)H, l.kv_heads, (int)d,
-                         (int)dv, T, m->t3, inner);
+            const float *x = m->t2, *Bv = x + inner, *Cv = Bv + GN, *dt = t1 + inner + P.cqkv;
+            if (T >= SSD_CHUNKED_FROM && !tiled && m->ssd_scratch && psk_ssd_chunked_ok((int)d, (int)dv))
+                psk_ssd_chunked(st, m->step, P.off_S, x, Bv, Cv, P.cqkv, dt, ld1, l.a_log, l.dt_bias, l.skip, (int)H, l.kv_heads, (int)d, (int)dv, T, m->ssd_scratch, m->t3, inner);
+            else
+                psk_ssd_scan(st, m->step, P.off_S, x, Bv, Cv, P.cqkv, dt, ld1, l.a_log, l.dt_bias, l.skip, (int)H, l.kv_heads, (int)d, (int)dv, T, m->t3, inner);
             psk_gate_partnorm(st, m->t3, inner, t1, ld1, l.onorm, l.norm_parts, D.norm_eps, inner, T);
             out_proj(m->t3, inner);
         } else if (l.kind == PS_MIX_MINGRU) {
