@@ -20,13 +20,13 @@ SOURCES = ["ctx.hip", "api.hip", "model.hip", "k_quant.hip", "k_gemv.hip", "k_ge
 # run did not come back within 15 minutes; the likeliest culprit is that run's CPU baseline leg -- the reference's spin-barrier thread pool on a busy
 # host, now a child process under a time limit in bench.py -- but the round had no GPU time left to tell the two apart, so every other file keeps the
 # exact compile configuration that has passed the full GPU suite and all bench configurations.)
-FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-Wno-unused-result",
+# -packed-fp32-ops: no file may use the packed fp32 instructions (v_pk_add_f32 and its like), whatever a compiler pass would make of ordinary float code.
+NO_PACKED = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-Wno-unused-result", *NO_PACKED,
          "-I" + os.path.join(HERE, "..", "include")]
 # The layer-list models (dense bf16 / fp32 matrices; include/ps_hip.h): their sources plus the context make a library of their own,
 # lib/libps_hip_seq.so, so that a checkout that only serves such a model compiles four files and not the quantized path's kernels.
 SEQ_SOURCES = ["ctx.hip", "seqmodel.hip", "k_dense.hip", "k_seqmix.hip", "k_latent.hip", "k_winattn.hip", "k_moe.hip", "k_ssd.hip"]
-# packed fp32 instructions are left to no one: these files are ordinary float code and are compiled without the feature
-SEQ_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 NOSLP = {"k_gemv4.hip", "k_qkvattn.hip", "k_gemvb.hip", "k_attn.hip", "k_gemm4k.hip"}  # k_gemm4k.hip (round 5): gate/up chunk launch of a 512-column sequence 384.2 -> 369-371 us, same bits (profiles/r05_g4k2_variants.txt, the "v2 0" lines vs profiles/r05_g4k_item_order.txt)  # (k_gemvb.hip: the Q4_0 / Q8_0 mat-vec, Llama-3.2-1B 1494 -> 1525 tok/s)
 
 
@@ -63,7 +63,7 @@ TIMELINE_SOURCES = {"api.hip", "k_gemv4.hip", "k_qkvattn.hip", "k_attn.hip", "k_
 
 
 def _compile_cmd(hipcc: str, s: str, src: str, obj: str) -> list:
-    return [hipcc, *FLAGS, *(["-fno-slp-vectorize"] if s in NOSLP else []), *(SEQ_FLAGS if s in SEQ_SOURCES and s != "ctx.hip" else []), "-c", src, "-o", obj]
+    return [hipcc, *FLAGS, *(["-fno-slp-vectorize"] if s in NOSLP else []), "-c", src, "-o", obj]
 
 
 def build_seq(force: bool = False, verbose: bool = True) -> str:

@@ -601,7 +601,7 @@ __global__ void dense_embed_kernel(const void *table, int is_bf16, long long K, 
 }
 void psk_embed(hipStream_t st, const ps_dense *table, const int32_t *tokens, const ps_seq_step *step, int T, float scale, float *out, int64_t ldo, const ps_dense *bigram,
                int64_t buckets, int64_t mul_prev, int64_t mul_cur) {
-    hipLaunchKernelGGL(dense_embed_kernel, dim3(T), dim3(256), 0, st, table->data, table->dtype == PS_BF16 ? 1 : 0, (long long)table->K, tokens, step, scale, out,
+    hipLaunchKernelGGL(dense_embed_kernel, dim3(T), dim3(T <= 8 && table->K >= 1024 ? 1024 : 256), 0, st, table->data, table->dtype == PS_BF16 ? 1 : 0, (long long)table->K, tokens, step, scale, out,
                        (long long)ldo, bigram ? bigram->data : nullptr, (long long)buckets, (long long)mul_prev, (long long)mul_cur);
 }
 
