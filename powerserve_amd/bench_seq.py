@@ -56,7 +56,7 @@ def config(z: dict, vocab: int = 4096) -> dict:
             own = max([j for j in range(i) if z["order"][j] == "a"], default=None)
             mixer = kinds.get(k) or ("attention", synth.pupidra_attention(H, z["kv_heads"], d, d, 1.0, z["window"], z["keep_first"], own if k == "s" else None))
             layers.append(synth.pupidra_layer(*mixer, moe=(z["experts"], z["top"], z["ff"] * 3 // 8, 2.0), shared=z["ff"] * 3 // 4))
-        return synth.pupidra_config(z["width"], vocab, layers, bigram=(4093, 31, 17), softcap=30.0)
+        return synth.pupidra_config(z["width"], vocab, layers, bigram=(4093, 43, 19), softcap=30.0)
     if z.get("design") == "Pokatar":
         att = synth.pokatar_attention(H, z["kv_heads"], d, d, float(d ** -0.5))
         lat = synth.pokatar_latent(H, d, z["rot_dim"], d, z["kv_rank"], float((d + z["rot_dim"]) ** -0.5), 5e5, (8.0, 4096, 16.0, 2.0))

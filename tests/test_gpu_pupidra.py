@@ -22,9 +22,9 @@ CONFIGS = {
                        UL("attention", UA(6, 1, 10, 6, 0.4, 17, 5, kv_from=1), (3, 3, 8, 1.0), 6), UL("mamba2", UM(4, 5, 12, 4, 1, 4)), UL("attention", UA(4, 4, 6, 10, 0.4, 12, 0)),
                        UL("attention", UA(4, 4, 6, 10, 0.2, 5, 1, kv_from=5), (5, 2, 12, 2.0))], bigram=(37, 5, 3), softcap=9.0, eps=1e-5),
     # sizes the matrix-core and chunked kernels take (inputs that are multiples of 64, state and value sizes that are multiples of 16)
-    "aligned": UC(128, 96, [UL("latent_attention", ULA(4, 48, 32, 16, 48, 0.15, 10000.0), (8, 2, 64, 2.5), 64), UL("mamba2", UM(8, 16, 32, 2, 4, 2), (6, 3, 64, 1.5), 128),
+    "aligned": UC(128, 96, [UL("latent_attention", ULA(4, 48, 32, 16, 48, 0.15, 10000.0), (8, 2, 64, 2.2), 64), UL("mamba2", UM(8, 16, 32, 2, 4, 2), (6, 3, 64, 1.5), 128),
                             UL("attention", UA(8, 2, 16, 32, 0.3, 24, 10), (4, 1, 128, 3.0), 64), UL("attention", UA(4, 2, 16, 32, 0.35, 40, 18, kv_from=2), (4, 2, 64, 1.0)),
-                            UL("mamba2", UM(4, 48, 64, 4, 2, 1), (8, 4, 64, 2.0), 64)], bigram=(211, 31, 17), softcap=12.0),
+                            UL("mamba2", UM(4, 48, 64, 4, 2, 1), (8, 4, 64, 2.0), 64)], bigram=(211, 29, 13), softcap=12.0),
     # a state of 160 over 6 heads in 3 groups, 20 heads on one key / value head, 18 latent heads; no bigram table, no soft cap
     "manyheads": UC(64, 40, [UL("mamba2", UM(6, 32, 160, 3, 4, 6)), UL("attention", UA(20, 1, 16, 8, 0.3, 30, 4), (2, 1, 16, 2.0), 16), UL("latent_attention", ULA(18, 16, 16, 8, 32, 0.2, 100.0), (3, 2, 32, 1.5))]),
     # 128 value columns per head, a latent wider than the model, the widest state the scan takes, heads == groups == 1
