@@ -313,6 +313,7 @@ enum ps_mixer_kind {
     PS_MIX_GLA    = 5, /* gated linear attention: S <- diag(alpha) S + k v^T, o = S^T q, a decay per key channel from a two-matrix projection */
     PS_MIX_MINGRU = 6, /* element-wise gated recurrence, its gates functions of the present input alone: S <- (1 - z) S + z c, output S * silu(g) */
     PS_MIX_SSD    = 7, /* state-space recurrence with one decay per head (Mamba-2): S <- exp(-exp(a_log) dt) S + dt B x^T, y = S^T C + D x, gated and normed in parts */
+    PS_MIX_MLSTM  = 8, /* matrix memory with exponential gates (mLSTM): S <- a S + b k v^T, n <- a n + b k under a running maximum, o = S^T q / max(|n . q|, exp(-m)) */
 };
 enum ps_ff_kind {
     PS_FF_NONE = 0,
@@ -328,7 +329,7 @@ enum ps_layer_form {
                               * not at all); h2 = h, or norm2(x) where norm2 is given (two weights over the same statistics) */
     PS_LAYER_PRENORM    = 2, /* x += mixer(norm1(x)), then x += ff(norm2(x)): the second norm reads what the mixer left; no input filter, nothing normed behind a sublayer */
     PS_LAYER_POSTNORM   = 3, /* x += norm1b(mixer(x)), then x += norm2b(ff(x)): the sublayers read the residual stream itself, only their outputs are normed (a layer scale is folded into
-                              * the norm's weight); no input filter, norm1 / norm2 unused */
+                              * the norm's weight, norm1b_bias / norm2b_bias are added behind it); no input filter, norm1 / norm2 unused */
 };
 enum ps_rot_pairing { PS_ROT_HALVES = 0 /* (i, i + dims/2) */, PS_ROT_NEIGHBOURS = 1 /* (2i, 2i + 1) */ };
 
@@ -405,7 +406,7 @@ typedef struct ps_seq_layer_s {
     /* gated == 2 (PS_MIX_WINATTN): the gate projection has heads * vdim rows and multiplies the concatenated heads element by element.
      * PS_MIX_LATENT reads gated too (1: a row per head; in_cat then ends with the gate's rows), and with q_rank == 0 its queries come straight from the input:
      *   in_cat = rows of q | dkv | gate ([heads * (dim + rot_dim) + kv_rank + rot_dim + (gated ? heads : 0), width]), uq and qnorm unused; window 0 = everything before the token */
-    /* ---- rotary frequency scaling by wavelength (PS_MIX_LATENT; yarn_factor 0: none): with dim(t) = rot_dims ln(yarn_original / (2 pi t)) / (2 ln rot_base),
+    /* ---- rotary frequency scaling by wavelength (PS_MIX_LATENT, PS_MIX_WINATTN; yarn_factor 0: none): with dim(t) = rot_dims ln(yarn_original / (2 pi t)) / (2 ln rot_base),
      * lo = max(floor(dim(yarn_fast)), 0), hi = min(ceil(dim(yarn_slow)), rot_dims - 1), ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), pair i turns with
      * f_i / yarn_factor * ramp_i + f_i (1 - ramp_i), and cos and sin are both multiplied by 0.1 ln(yarn_factor) + 1 */
     float yarn_factor, yarn_fast, yarn_slow;
@@ -413,7 +414,8 @@ typedef struct ps_seq_layer_s {
     /* ---- feed-forward extras */
     const float *ff_up_bias, *ff_down_bias; /* PS_FF_DENSE_RELU_GLU / PS_FF_DENSE_SWIGLU: biases of the (interleaved) gate / up rows and of the down rows, or NULL */
     /* mixtures of experts: `experts` counts the feed-forwards that have tensors; the router has experts + moe_identity rows, the last moe_identity of which are
-     * identity experts (their output is their input).  moe_softmax 1: scores = soft-max over all router rows (0: sigmoid).  moe_correction [router rows] or NULL is added
+     * identity experts (their output is their input).  moe_softmax 1: scores = soft-max over all router rows (0: sigmoid); 2: the
+     * largest LOGITS are chosen and a chosen row's weight is its share of the soft-max over the chosen ones alone.  moe_correction [router rows] or NULL is added
      * to the scores for the CHOICE only.  moe_groups > 0: the router rows form that many equal groups of neighbours, a group's score is its largest choice score, and
      * only rows of the moe_keep best groups can be chosen.  moe_weight_output 1: a chosen expert's score multiplies its output (0: its input). */
     int32_t moe_identity, moe_softmax, moe_groups, moe_keep, moe_weight_output;
@@ -434,6 +436,21 @@ typedef struct ps_seq_layer_s {
      *   dt = softplus(dt + dt_bias); the result times silu(z) is RMS-normed in norm_parts equal stretches, times onorm */
     int32_t norm_parts;
     const float *conv_bias, *skip;      /* skip: D [heads] */
+    /* ---- post-norm layers, continued */
+    const float *norm1b_bias, *norm2b_bias; /* [width] added behind norm1b / norm2b, or NULL */
+    const float *mix_onorm;             /* [width] or NULL: the mixer's output is divided by its root mean square over the width and multiplied by this, in front of mix_scale and of the sum
+                                         * of two mixers side by side (either both have it or none) */
+    /* ---- mixtures of experts, continued */
+    const float *router_bias;           /* [router rows] added to the router's logits, or NULL */
+    /* ---- per-layer token input (post-norm layers), behind the feed-forward: with e the layer's side_dim numbers of the token's row of ps_seq_desc::side_embed,
+     * x += rms(side_proj (gelu(side_gate x) * e)) * side_norm (an RMS norm with a plain weight, gelu in its tanh form).  side_gate [side_dim, width], side_proj [width, side_dim]; NULL: none */
+    const ps_dense *side_gate, *side_proj;
+    const float *side_norm;
+    /* ---- PS_MIX_MLSTM; it reads heads, dim, vdim, onorm [heads * vdim], out.
+     *   in_cat = rows of q | k | v | g | i | f  ([2*heads*dim + 2*heads*vdim + 2*heads, width]), in_bias [rows of in_cat] or NULL; q is scaled by dim^-1/2; with c(z) = gate_cap tanh(z / gate_cap)
+     *   log input gate c(i), log forget gate ln sigmoid(c(f)); m <- max(f + m, i) from m = 0, S <- exp(f + m_old - m) S + exp(i - m) k v^T, n alike with k alone;
+     *   o = S^T q / (max(|n . q|, exp(-m)) + 1e-6), each head divided by its root mean square, times onorm, times sigmoid(g) */
+    float gate_cap;                     /* 0: gates as they are */
 } ps_seq_layer;
 
 typedef struct {
@@ -451,12 +468,15 @@ typedef struct {
     int32_t loop_start, loop_stop, loop_times;
     int32_t max_context; /* most tokens a sequence may hold: sizes what grows with a sequence (the pooled blocks of PS_MIX_WINATTN, a window of everything); 0: 65536 */
     int32_t norm_groups; /* every RMS norm over the width is taken in this many equal consecutive parts, each with its own mean square (0 is taken as 1) */
-    int32_t norm_center; /* 1: the norms over the width are layer norms -- the mean is taken off first and the variance is the mean of the squared deviations (PS_LAYER_PRENORM layers and the final norm) */
+    int32_t norm_center; /* 1: the norms over the width are layer norms -- the mean is taken off first and the variance is the mean of the squared deviations (PS_LAYER_PRENORM and PS_LAYER_POSTNORM layers and the final norm; side_norm and mix_onorm stay RMS norms) */
     /* a second embedding table [bigram_buckets + 1, width], or NULL: row (previous token * bigram_mul_prev + token * bigram_mul_cur) mod bigram_buckets is added to the token's
      * embedding, the last row for a sequence's first token (the previous token is part of a sequence's state) */
     const ps_dense *bigram;
     int64_t bigram_buckets, bigram_mul_prev, bigram_mul_cur;
     float logit_softcap; /* logits <- logit_softcap * tanh(logits / logit_softcap), before logit_scale (0: none) */
+    int32_t side_dim;    /* per-layer token input: numbers per layer in a row of side_embed */
+    const ps_dense *side_embed; /* [vocab, n_layers * side_dim] or NULL; layer i reads numbers i side_dim .. (i + 1) side_dim - 1 of the token's row */
+    const float *final_norm_bias; /* [width] added behind the final norm, or NULL */
 } ps_seq_desc;
 
 int ps_hip_seq_create(ps_hip_ctx *ctx, const ps_seq_desc *desc, ps_hip_seq **out);

@@ -197,8 +197,19 @@ std::vector<float> expect1(const SafeTensorsFile &st, const std::string &n, int6
     if (t.shape.size() != 1 || t.shape[0] != r) POWERSERVE_ABORT("tensor " + n + ": its shape is not what the configuration gives");
     return st.f32(n);
 }
-// windowed attention with pooled blocks: whatever the configuration or the file does not have does not exist
-void window_attention_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &m, const JsonValue &mc) {
+// rotary frequencies scaled by wavelength, where the configuration's rot has a 'scaling'
+void wavelength_scaling(ps_seq_layer &L, const JsonValue &rot) {
+    if (const JsonValue *sc = obj_or_null(rot, "scaling")) {
+        L.yarn_factor = (float)sc->at("factor").num;
+        L.yarn_fast = (float)sc->at("fast").num;
+        L.yarn_slow = (float)sc->at("slow").num;
+        L.yarn_original = (int32_t)sc->at("original").num;
+    }
+}
+// windowed attention with pooled blocks: whatever the configuration or the file does not have does not exist.  by_wavelength: rot.scaling scales the frequencies by wavelength
+// (else all of them by its factor)
+void window_attention_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &m, const JsonValue &mc, int pairing = PS_ROT_NEIGHBOURS,
+                            bool by_wavelength = false) {
     L.kind = PS_MIX_WINATTN;
     L.heads = (int32_t)mc.at("heads").num;
     L.dim = (int32_t)mc.at("dim").num;
@@ -206,13 +217,14 @@ void window_attention_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploa
     L.vdim = (int32_t)num_or(mc, "vdim", L.dim);
     if (L.kv_heads <= 0 || L.heads % L.kv_heads) POWERSERVE_ABORT(m + ": heads must be a multiple of kv_heads");
     if (const JsonValue *mask = obj_or_null(mc, "mask")) { L.window = (int32_t)num_or(*mask, "size", 0); L.pool = (int32_t)num_or(*mask, "pool", 0); }
-    L.rot_pairing = PS_ROT_NEIGHBOURS;
+    L.rot_pairing = pairing;
     L.rot_base = 10000.f;
     L.rot_factor = 1.f;
     if (const JsonValue *rot = obj_or_null(mc, "rot")) {
         L.rot_dims = (int32_t)num_or(*rot, "dims", 0);
         L.rot_base = (float)num_or(*rot, "base", 10000.0);
-        if (const JsonValue *sc = obj_or_null(*rot, "scaling")) L.rot_factor = (float)num_or(*sc, "factor", 1.0);
+        if (by_wavelength) wavelength_scaling(L, *rot);
+        else if (const JsonValue *sc = obj_or_null(*rot, "scaling")) L.rot_factor = (float)num_or(*sc, "factor", 1.0);
     }
     L.scale = (float)num_or(mc, "scale", 1.0 / std::sqrt((double)L.dim));
     L.softcap = (float)num_or(mc, "softcap", 0.0);
@@ -338,7 +350,8 @@ void append_gate_up(const SafeTensorsFile &st, const std::string &p, int64_t ff,
         memcpy(&all[at + (size_t)(2 * r + 1) * W], &u[(size_t)r * W], (size_t)W * 2);
     }
 }
-void gated_feed_forward(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &p, const JsonValue &f, int64_t W) {
+// chosen_softmax: the largest logits are chosen and their soft-max weighs the experts' outputs (else a chosen expert's sigmoid score weighs its input)
+void gated_feed_forward(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &p, const JsonValue &f, int64_t W, bool chosen_softmax = false) {
     const std::string kind = f.at("kind").str;
     if (kind == "dense") {
         L.ff_kind = PS_FF_DENSE_SWIGLU;
@@ -363,6 +376,8 @@ void gated_feed_forward(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader 
         L.ff_up = up.mat(ups, (int64_t)L.experts * 2 * L.ff, W);
         L.ff_down = up.mat(downs, (int64_t)L.experts * W, L.ff);
         L.router = up.vec(expect(st, p + "router", L.experts, W));
+        if (st.contains(p + "router.b")) L.router_bias = up.vec(expect1(st, p + "router.b", L.experts));
+        if (chosen_softmax) { L.moe_softmax = 2; L.moe_weight_output = 1; }
         if (const JsonValue *sh = obj_or_null(f, "shared")) {
             L.shared_ff = (int32_t)sh->at("ff").num;
             std::vector<uint16_t> both;
@@ -455,12 +470,7 @@ void shared_key_latent_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUplo
     if (const JsonValue *rot = obj_or_null(mc, "rot")) {
         L.rot_dims = (int32_t)num_or(*rot, "dims", 0);
         L.rot_base = (float)num_or(*rot, "base", 10000.0);
-        if (const JsonValue *sc = obj_or_null(*rot, "scaling")) {
-            L.yarn_factor = (float)sc->at("factor").num;
-            L.yarn_fast = (float)sc->at("fast").num;
-            L.yarn_slow = (float)sc->at("slow").num;
-            L.yarn_original = (int32_t)sc->at("original").num;
-        }
+        wavelength_scaling(L, *rot);
     }
     if (const JsonValue *mask = obj_or_null(mc, "mask")) L.window = (int32_t)num_or(*mask, "size", 0);
     L.scale = (float)mc.at("scale").num;
@@ -680,10 +690,89 @@ void pupidra(const JsonValue &cfg, const SafeTensorsFile &st, SeqUploader &up, s
         layers.push_back(L);
     }
 }
+// ---------------------------------------------------------------- Sogavik: post-norm layers with biased layer norms, windowed attention alone or beside a matrix memory, a token input per layer
+void matrix_memory_mixer(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &m, const JsonValue &mc) {
+    L.kind = PS_MIX_MLSTM;
+    L.heads = (int32_t)mc.at("heads").num;
+    L.dim = (int32_t)mc.at("dim").num;
+    L.vdim = (int32_t)num_or(mc, "vdim", L.dim);
+    L.gate_cap = (float)num_or(mc, "gate_cap", 0.0);
+    const int64_t Hd = (int64_t)L.heads * L.dim, Hv = (int64_t)L.heads * L.vdim;
+    std::vector<std::string> names;
+    for (const auto &[n, r] : std::vector<std::pair<std::string, int64_t>>{{"q", Hd}, {"k", Hd}, {"v", Hv}, {"g", Hv}, {"i", L.heads}, {"f", L.heads}}) {
+        check_rows(st, m + n, r);
+        names.push_back(m + n);
+    }
+    L.in_cat = mat_rows(st, up, names);
+    bool any = false;
+    const auto bias = stacked_bias(st, names, any);
+    if (any) L.in_bias = up.vec(bias);
+    L.onorm = up.vec(expect1(st, m + "norm", Hv));
+    L.out = mat1(st, up, m + "o");
+}
+void token_side_input(ps_seq_layer &L, const SafeTensorsFile &st, SeqUploader &up, const std::string &p, int64_t dim, int64_t W) {
+    check_rows(st, p + "gate", dim);
+    check_rows(st, p + "proj", W);
+    L.side_gate = mat1(st, up, p + "gate");
+    L.side_proj = mat1(st, up, p + "proj");
+    L.side_norm = up.vec(expect1(st, p + "norm", W));
+}
+void sogavik(const JsonValue &cfg, const SafeTensorsFile &st, SeqUploader &up, std::vector<ps_seq_layer> &layers, ps_seq_desc &d) {
+    d.width = (int32_t)cfg.at("width").num;
+    d.vocab = (int32_t)cfg.at("vocab").num;
+    d.canon_taps = 1;
+    d.norm_eps = (float)cfg.at("norm").at("eps").num;
+    d.norm_offset = 0.0f;
+    d.norm_center = 1;
+    d.logit_scale = 1.0f;
+    d.loop_times = 1;
+    auto bias_of = [&](const std::string &n) -> const float * { return st.contains(n + ".b") ? up.vec(expect1(st, n + ".b", d.width)) : nullptr; };
+    d.embed = mat1(st, up, "embed");
+    d.head = mat1(st, up, "head");
+    d.final_norm = up.vec(expect1(st, "final.norm", d.width));
+    d.final_norm_bias = bias_of("final.norm");
+    const auto &ls = cfg.at("layers").arr;
+    if (const JsonValue *side = obj_or_null(cfg, "token_side")) {
+        d.side_dim = (int32_t)side->at("dim").num;
+        if (cols_of(st, "side.embed") != (int64_t)ls.size() * d.side_dim) POWERSERVE_ABORT("tensor side.embed: its shape is not what the configuration gives");
+        check_rows(st, "side.embed", d.vocab);
+        d.side_embed = mat1(st, up, "side.embed");
+    }
+    for (size_t i = 0; i < ls.size(); i++) {
+        const JsonValue &lc = ls[i], &mc = lc.at("mixer");
+        const std::string p = "l" + std::to_string(i) + ".", m = p + "mix.", kind = lc.at("type").str;
+        ps_seq_layer L{};
+        L.form = PS_LAYER_POSTNORM;
+        L.mix_scale = 1.f;
+        L.norm1b = up.vec(expect1(st, p + "norm1", d.width));
+        L.norm1b_bias = bias_of(p + "norm1");
+        if (kind == "attention") {
+            window_attention_mixer(L, st, up, m, mc, PS_ROT_HALVES, true);
+        } else if (kind == "parallel") {
+            ps_seq_layer R{};
+            window_attention_mixer(L, st, up, m + "left.", mc.at("left"), PS_ROT_HALVES, true);
+            matrix_memory_mixer(R, st, up, m + "right.", mc.at("right"));
+            L.mix_onorm = up.vec(expect1(st, m + "left.out", d.width));
+            R.mix_onorm = up.vec(expect1(st, m + "right.out", d.width));
+            L.mix_scale = R.mix_scale = 0.5f;
+            up.beside.push_back(R);
+            L.beside = &up.beside.back();
+        } else {
+            POWERSERVE_ABORT("layer " + std::to_string(i) + ": mixer type " + kind + " is not known");
+        }
+        if (lc.contains("mlp") && lc.at("mlp").kind == JsonValue::OBJ) {
+            L.norm2b = up.vec(expect1(st, p + "norm2", d.width));
+            L.norm2b_bias = bias_of(p + "norm2");
+            gated_feed_forward(L, st, up, p + "mlp.", lc.at("mlp"), d.width, true);
+        }
+        if (d.side_embed) token_side_input(L, st, up, p + "side.", d.side_dim, d.width);
+        layers.push_back(L);
+    }
+}
 } // namespace
 
 const std::map<std::string, SeqArchitecture> &seq_architectures() {
-    static const std::map<std::string, SeqArchitecture> reg = {{"Ranutar", ranutar}, {"Vobisun", vobisun}, {"Zusolix", zusolix}, {"Pokatar", pokatar}, {"Pupidra", pupidra}};
+    static const std::map<std::string, SeqArchitecture> reg = {{"Ranutar", ranutar}, {"Vobisun", vobisun}, {"Zusolix", zusolix}, {"Pokatar", pokatar}, {"Pupidra", pupidra}, {"Sogavik", sogavik}};
     return reg;
 }
 bool is_seq_model_dir(const std::string &dir) {

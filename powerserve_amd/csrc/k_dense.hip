@@ -4,7 +4,7 @@
 //   dense_mm_fast_kernel  bf16, K % 64 == 0, more than 8 tokens: 128 x 128 tiles over an operand packed to bf16 by dense_pack_kernel
 //   dense_mv_kernel<WT,C> a few tokens (C <= 8 columns): the activation rows live in LDS, a wave streams four weight rows at a time
 // All take the same operand description (ps_seq.h psk_dense_args): ring rows, the token-shift mix and the epilogue
-// (bias, xIELU / tanh, scale) are part of the launch, so no mixer needs a kernel of its own around its projections.
+// (bias, activation, scale, a factor from a second table) are part of the launch, so no mixer needs a kernel of its own around its projections.
 #include "ps_seq.h"
 
 #include <cmath>
@@ -43,6 +43,11 @@ struct dn_args {
     long long wstride;
     const float *g_ident, *g_ident_w; // grouped mat-vec: a slot without a matrix adds g_ident_w[slot] * g_ident[row][n] to output n
     long long g_ident_ld;
+    const void *em_table; // a factor per output from the token's row of a second table (psk_dense_args)
+    int em_bf16;
+    long long em_ld, em_col;
+    const int32_t *em_tokens;
+    const ps_seq_step *em_step;
 };
 
 // rows of A that exist and where they start (ring rows relative to the step's position)
@@ -85,6 +90,8 @@ static __device__ __forceinline__ float dn_epi(const dn_args &g, float acc, long
         acc = acc > 0.f ? acc * acc : 0.f;
     } else if (g.act == PSD_ACT_SOFTCAP) {
         acc = g.act_p * tanhf(acc / g.act_p);
+    } else if (g.act == PSD_ACT_GELU_TANH) {
+        acc = 0.5f * acc * (1.f + tanhf(0.7978845608028654f * (acc + 0.044715f * acc * acc * acc)));
     }
     return acc * g.alpha;
 }
@@ -104,7 +111,11 @@ static __device__ __forceinline__ void dn_put(const dn_args &g, long long t, lon
     }
     if (!in) return;
     float *p = g.out + t * g.ldo + n;
-    const float v = dn_epi(g, acc, n) * rs;
+    float v = dn_epi(g, acc, n) * rs;
+    if (g.em_table) {
+        const long long at = (long long)(g.em_tokens ? g.em_tokens[t] : g.em_step->token0) * g.em_ld + g.em_col + n;
+        v *= g.em_bf16 ? dn_bf2f(((const unsigned short *)g.em_table)[at]) : ((const float *)g.em_table)[at];
+    }
     *p = g.accum ? *p + v : v;
 }
 // the output row of local row t (t < T): itself, or where the sorted list sends its slot
@@ -505,6 +516,8 @@ int psk_dense(hipStream_t st, const psk_dense_args &a) {
     g.alpha = a.alpha; g.mu = a.mu; g.shift0 = a.shift0; g.accum = a.accum; g.out_scale = a.out_scale;
     g.groups = 0; g.g_adiv = 1; g.g_odiv = 1; g.g_inner = 1; g.g_sel = nullptr; g.g_seg = nullptr; g.g_list = nullptr; g.g_scale = nullptr; g.wstride = 0;
     g.g_ident = a.g_ident; g.g_ident_w = a.g_ident_w; g.g_ident_ld = a.g_ident_ld;
+    g.em_table = a.em_table ? a.em_table->data : nullptr; g.em_bf16 = a.em_table && a.em_table->dtype == PS_BF16; g.em_ld = a.em_table ? a.em_table->K : 0;
+    g.em_col = a.em_col; g.em_tokens = a.em_tokens; g.em_step = a.em_step;
     const bool bf = a.w->dtype == PS_BF16;
     const size_t kp4 = (size_t)((g.K + 7) / 8 * 8) * 4;
     if (a.groups > 0) {

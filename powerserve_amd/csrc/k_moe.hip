@@ -1,7 +1,7 @@
 // Mixture-of-experts routing for the layer-list models (PS_FF_MOE_SWIGLU, PS_FF_MOE_RELU2).  The experts' matrix products are grouped launches of the dense kernels
 // (k_dense.hip); here is what decides who goes where, all fp32:
-//   moe_route_kernel    a block per token: router logits, sigmoid or soft-max scores, a correction and a group limit on the choice, the `top` largest
-//                       (their scores times a constant), the shared expert's gate
+//   moe_route_kernel    a block per token: router logits (+ bias), sigmoid or soft-max scores, a correction and a group limit on the choice, the `top` largest
+//                       (their scores, or the soft-max over the chosen logits alone, times a constant), the shared expert's gate
 //   moe_plan_kernel     the token-expert slots sorted by expert (counts, offsets, list) for the tiled products
 //   moe_combine_kernel  a token's `top` per-slot results summed into the residual stream; an identity expert's share is its weight times the input
 #include "ps_seq.h"
@@ -22,7 +22,7 @@ typedef float moe_f4 __attribute__((ext_vector_type(4)));
 // dynamic LDS: [rows + 1] scores, [rows] choice scores, [groups] group scores.
 __global__ __launch_bounds__(256) void moe_route_kernel(const float *h, long long ldh, const float *router, const float *shared_gate, int experts, int top, int norm_top,
                                                         long long K, int softmax, const float *correction, int n_groups, int keep, float scale, int32_t *sel,
-                                                        float *wgt, float *sgate) {
+                                                        float *wgt, float *sgate, const float *bias) {
     extern __shared__ float sc[];
     float *ch = sc + experts + 1, *gs = ch + experts;
     const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -52,12 +52,13 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float *h, long lon
             for (long long k = lane; k < K; k += 64) a = fmaf(w[k], x[k], a);
         }
         a = moe_wave_sum(a);
+        if (bias && e < experts) a += bias[e];
         if (lane == 0) sc[e] = softmax && e < experts ? a : moe_sigmoid(a);
     }
     __syncthreads();
     if (wave) return;
     if (shared_gate && lane == 0) sgate[t] = sc[experts];
-    if (softmax) {
+    if (softmax == 1) {
         float mx = -INFINITY, sum = 0.f;
         for (int e = lane; e < experts; e += 64) mx = fmaxf(mx, sc[e]);
 #pragma unroll
@@ -110,19 +111,27 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float *h, long lon
             if (ch[e] > best) { best = ch[e]; at = e; }
         agree(best, at);
         const bool any = at != 0x7fffffff; // (nothing left in the race: the slot goes to row 0 with weight 0)
-        const float w = any ? sc[at] : 0.f;
-        if (lane == 0) { sel[(long long)t * top + i] = any ? at : 0; wgt[(long long)t * top + i] = norm_top ? w : w * scale; if (any) ch[at] = -INFINITY; }
+        const float w = any ? sc[at] : softmax == 2 ? -INFINITY : 0.f;
+        if (lane == 0) { sel[(long long)t * top + i] = any ? at : 0; wgt[(long long)t * top + i] = norm_top || softmax == 2 ? w : w * scale; if (any) ch[at] = -INFINITY; }
         total += w;
         __builtin_amdgcn_wave_barrier();
         __threadfence_block();
     }
-    if (norm_top)
+    if (softmax == 2) { // the soft-max over the chosen logits
+        float mx = -INFINITY, sum = 0.f;
+        for (int i = lane; i < top; i += 64) mx = fmaxf(mx, wgt[(long long)t * top + i]);
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
+        for (int i = lane; i < top; i += 64) sum += expf(wgt[(long long)t * top + i] - mx);
+        sum = moe_wave_sum(sum);
+        for (int i = lane; i < top; i += 64) wgt[(long long)t * top + i] = expf(wgt[(long long)t * top + i] - mx) / sum * scale;
+    } else if (norm_top)
         for (int i = lane; i < top; i += 64) wgt[(long long)t * top + i] = wgt[(long long)t * top + i] / total * scale;
 }
 void psk_moe_route(hipStream_t st, const float *h, int64_t ldh, const float *router, const float *shared_gate, int experts, int top, int norm_top, int64_t K, int T,
-                   int32_t *sel, float *wgt, float *sgate, int softmax, const float *correction, int n_groups, int keep, float scale) {
+                   int32_t *sel, float *wgt, float *sgate, int softmax, const float *correction, int n_groups, int keep, float scale, const float *bias) {
     hipLaunchKernelGGL(moe_route_kernel, dim3(T), dim3(256), (size_t)(2 * experts + 1 + (n_groups > 0 ? n_groups : 0)) * 4, st, h, (long long)ldh, router, shared_gate,
-                       experts, top, norm_top, (long long)K, softmax, correction, n_groups, keep, scale, sel, wgt, sgate);
+                       experts, top, norm_top, (long long)K, softmax, correction, n_groups, keep, scale, sel, wgt, sgate, bias);
 }
 
 // one block; dynamic LDS: 2 x experts ints.  Counts, offsets, then every slot takes the next free place of its expert.  Which place a slot gets is up to the

@@ -1,5 +1,5 @@
 // Mechanisms of the layer-list models that are not matrix products: RMS norms (with the residual add), causal convolutions over time
-// with a per-sequence tail, and the recurrent scans (wkv, gated linear attention, gated delta rule, state space, element-wise).  Everything here is fp32.
+// with a per-sequence tail, and the recurrent scans (wkv, gated linear attention, gated delta rule, state space, matrix memory, element-wise).  Everything here is fp32.
 //
 // The scans: a head's state S [d][dv] is split by COLUMN over threads -- every column j evolves on its own in both recurrences
 // (S_ij <- decay S_ij + k_i x_j needs only column j) -- and each column over R lanes of 16 rows each, so a step is 16 fused
@@ -46,7 +46,8 @@ void psk_rmsnorm(hipStream_t st, const float *x, int64_t ldx, const int32_t *idx
 // center: a layer norm instead -- the part's mean is taken off and the variance is the mean of the squared deviations (two passes over the row in LDS).
 // dynamic LDS: n + 2 groups floats.
 __global__ __launch_bounds__(1024) void sq_front_kernel(const float *src, long long stride, int nmix, const float *mix, const int32_t *idx, float *xout, const float *w1,
-                                                       float *h, const float *w2, float *h2, int groups, float offset, float eps, long long n, int center) {
+                                                       float *h, const float *w2, float *h2, int groups, float offset, float eps, long long n, int center,
+                                                       const float *bias) {
     extern __shared__ float fr[];
     float *xs = fr, *inv = fr + n, *mean = inv + groups;
     const long long r = idx ? idx[blockIdx.x] : blockIdx.x, o = (long long)blockIdx.x * n;
@@ -82,17 +83,17 @@ __global__ __launch_bounds__(1024) void sq_front_kernel(const float *src, long l
     __syncthreads();
     for (long long i = tid; i < n; i += nt) {
         const float v = (xs[i] - mean[i / gs]) * inv[i / gs];
-        if (w1) h[o + i] = v * (offset + w1[i]);
+        if (w1) h[o + i] = v * (offset + w1[i]) + (bias ? bias[i] : 0.f);
         if (w2) h2[o + i] = v * (offset + w2[i]);
     }
 }
 void psk_front(hipStream_t st, const float *src, int64_t stride, int nmix, const float *mix, const int32_t *idx, float *xout, const float *w1, float *h, const float *w2,
-               float *h2, int groups, float offset, float eps, int64_t n, int rows, int center) {
+               float *h2, int groups, float offset, float eps, int64_t n, int rows, int center, const float *bias) {
     if (rows <= 0) return;
     static unsigned long long mask = 0;
     if (ps_first_on_device(&mask)) (void)hipFuncSetAttribute((const void *)sq_front_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
     hipLaunchKernelGGL(sq_front_kernel, dim3(rows), dim3(rows <= 8 && n >= 2048 ? 1024 : 256), (size_t)(n + 2 * groups) * 4, st, src, (long long)stride, nmix, mix, idx, xout, w1, h, w2, h2, groups, offset, eps,
-                       (long long)n, center);
+                       (long long)n, center, bias);
 }
 
 __global__ __launch_bounds__(256) void sq_norm_residual_kernel(float *x, const float *y, const float *w, float offset, float eps, long long n) {
@@ -110,6 +111,55 @@ __global__ __launch_bounds__(256) void sq_norm_residual_kernel(float *x, const f
 void psk_norm_residual(hipStream_t st, float *x, const float *y, const float *w, float offset, float eps, int64_t n, int rows, int groups) {
     if (rows <= 0) return;
     hipLaunchKernelGGL(sq_norm_residual_kernel, dim3(rows, groups), dim3(256), 0, st, x, y, w, offset, eps, (long long)(n / groups));
+}
+
+// x += norm(v) (offset + w) + bias: a post-norm sublayer's end (ps_seq.h psk_postnorm), a block per row.  v = y, or the weighted sum of two outputs each divided by its own root mean
+// square; it stays in LDS between the passes (a thread re-reads what it wrote).  dynamic LDS: n floats.
+__global__ __launch_bounds__(1024) void sq_postnorm_kernel(float *x, const float *y, const float *w1, float s1, const float *y2, const float *w2, float s2, const float *w,
+                                                           const float *bias, float offset, int center, float eps, long long n) {
+    extern __shared__ float vs[];
+    __shared__ float red[2][16];
+    const int tid = threadIdx.x, nt = blockDim.x;
+    const long long at = (long long)blockIdx.x * n;
+    float *xr = x + at;
+    const float *a = y + at, *b = y2 ? y2 + at : nullptr;
+    auto block_sums = [&](float &p, float &q) { // both over the whole block
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) { p += __shfl_xor(p, o, 64); q += __shfl_xor(q, o, 64); }
+        __syncthreads();
+        if ((tid & 63) == 0) { red[0][tid >> 6] = p; red[1][tid >> 6] = q; }
+        __syncthreads();
+        p = q = 0.f;
+        for (int k = 0; k < (nt >> 6); k++) { p += red[0][k]; q += red[1][k]; }
+    };
+    float sum = 0.f, unused = 0.f;
+    if (w1) {
+        float p = 0.f, q = 0.f;
+        for (long long i = tid; i < n; i += nt) { p += a[i] * a[i]; if (b) q += b[i] * b[i]; }
+        block_sums(p, q);
+        const float ip = s1 / sqrtf(p / (float)n + eps), iq = s2 / sqrtf(q / (float)n + eps);
+        for (long long i = tid; i < n; i += nt) {
+            const float v = a[i] * ip * w1[i] + (b ? b[i] * iq * w2[i] : 0.f);
+            vs[i] = v;
+            sum += v;
+        }
+    } else {
+        for (long long i = tid; i < n; i += nt) { const float v = a[i]; vs[i] = v; sum += v; }
+    }
+    float mu = 0.f;
+    if (center) { block_sums(sum, unused); mu = sum / (float)n; }
+    float ss = 0.f;
+    for (long long i = tid; i < n; i += nt) { const float dv = vs[i] - mu; ss += dv * dv; }
+    block_sums(ss, unused);
+    const float inv = 1.f / sqrtf(ss / (float)n + eps);
+    for (long long i = tid; i < n; i += nt) xr[i] += (vs[i] - mu) * inv * (offset + w[i]) + (bias ? bias[i] : 0.f);
+}
+void psk_postnorm(hipStream_t st, float *x, const float *y, const float *w1, float s1, const float *y2, const float *w2, float s2, const float *w, const float *bias, float offset,
+                  int center, float eps, int64_t n, int rows) {
+    if (rows <= 0) return;
+    static unsigned long long mask = 0;
+    if (ps_first_on_device(&mask)) (void)hipFuncSetAttribute((const void *)sq_postnorm_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
+    hipLaunchKernelGGL(sq_postnorm_kernel, dim3(rows), dim3(rows <= 8 && n >= 2048 ? 1024 : 256), (size_t)n * 4, st, x, y, w1, s1, y2, w2, s2, w, bias, offset, center, eps, (long long)n);
 }
 
 // ---------------------------------------------------------------------------------------------------- causal convolution with a tail
@@ -626,6 +676,179 @@ void psk_ssd_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, co
     const int cols = two ? 2 * cpb : cpb;
     hipLaunchKernelGGL(kernel, dim3((P + cols - 1) / cols, H), dim3(256), lds, st, step, (long long)state_off, x, B, C, (long long)ld, dtraw, (long long)ldb, a_log, dt_bias, skip,
                        H, G, N, P, R, T, o, (long long)ldo);
+}
+
+// ---------------------------------------------------------------------------------------------------- matrix memory with exponential gates (mLSTM)
+static __device__ __forceinline__ float sq_capped(float z, float cap) { return cap > 0.f ? cap * tanhf(z / cap) : z; }
+static __device__ __forceinline__ float sq_log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
+// The scan of the state-space recurrence above with the gates of psk_mlstm_scan and one column more: column P has the value 1 for every token, which makes it n.  Every block walks the
+// running maximum for itself (wave 0, a lane per token of the round); the block with column P keeps it for the launch behind.
+// LDS: cs, bs [TC][dp]; per token: decay, input weight
+template <int NC>
+__global__ __launch_bounds__(256) void sq_mlstm_scan_kernel(const ps_seq_step *step, long long state_off, long long m_off, const float *q, const float *k, const float *v, long long ld,
+                                                            const float *iraw, const float *fraw, long long ldb, float cap, float qscale, int H, int N, int P, int R, int T, float *o,
+                                                            long long ldo, float *nq, float *mt) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    const int dp = SQ_NR * R, cpb = 256 / R;
+    float *cs = lds, *bs = cs + SQ_TC * dp, *gs = bs + SQ_TC * dp, *ds = gs + SQ_TC;
+    const int h = blockIdx.y, tid = threadIdx.x, s = tid % R, j0 = blockIdx.x * cpb * NC + tid / R;
+    const bool vec = N % 16 == 0, last = (int)(blockIdx.x + 1) * cpb * NC > P; // (last: this block has column P)
+    float *S0 = step->state + state_off + (long long)h * (P + 1) * N;
+    float S[NC][SQ_NR];
+#pragma unroll
+    for (int c = 0; c < NC; c++) {
+        const int j = j0 + c * cpb;
+        const float *Sj = S0 + (long long)j * N + s * SQ_NR;
+        if (vec) {
+            const bool in = j <= P && s * SQ_NR < N;
+#pragma unroll
+            for (int m4 = 0; m4 < SQ_NR / 4; m4++) {
+                const sq_f4 x = in ? *(const sq_f4 *)(Sj + 4 * m4) : sq_f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int e = 0; e < 4; e++) S[c][4 * m4 + e] = x[e];
+            }
+        } else {
+#pragma unroll
+            for (int m = 0; m < SQ_NR; m++) S[c][m] = (j <= P && s * SQ_NR + m < N) ? Sj[m] : 0.f;
+        }
+    }
+    const long long nb = (long long)h * N, vb = (long long)h * P;
+    float mrun = step->state[m_off + h];
+    float pa[SQ_PF], pb[SQ_PF], pv[NC][SQ_TC], pi = 0.f, pf = 0.f;
+    auto fetch = [&](int t0) {
+        const int nt = min(SQ_TC, T - t0);
+#pragma unroll
+        for (int e = 0; e < SQ_PF; e++) {
+            const int i0 = tid + 256 * e, t = i0 / dp, i = i0 % dp;
+            const bool in = i0 < SQ_TC * dp && t < nt && i < N;
+            const long long at = (long long)(t0 + (in ? t : 0)) * ld + nb + (in ? i : 0);
+            pa[e] = in ? q[at] : 0.f;
+            pb[e] = in ? k[at] : 0.f;
+        }
+        if (tid < 64) {
+            const bool in = tid < nt;
+            pi = in ? iraw[(long long)(t0 + tid) * ldb + h] : 0.f;
+            pf = in ? fraw[(long long)(t0 + tid) * ldb + h] : 0.f;
+        }
+#pragma unroll
+        for (int c = 0; c < NC; c++)
+#pragma unroll
+            for (int t = 0; t < SQ_TC; t++) {
+                const int j = j0 + c * cpb;
+                pv[c][t] = t >= nt ? 0.f : j < P ? v[(long long)(t0 + t) * ld + vb + j] : j == P ? 1.f : 0.f;
+            }
+    };
+    fetch(0);
+    for (int t0 = 0; t0 < T; t0 += SQ_TC) {
+        const int nt = min(SQ_TC, T - t0);
+        __syncthreads();
+#pragma unroll
+        for (int e = 0; e < SQ_PF; e++) {
+            const int i0 = tid + 256 * e;
+            if (i0 < SQ_TC * dp) {
+                cs[i0] = pa[e] * qscale;
+                bs[i0] = pb[e];
+            }
+        }
+        if (tid < 64) {
+            // (a token that is not there: forget gate 1, input gate 0 -- maximum and state stay)
+            const float li = tid < nt ? sq_capped(pi, cap) : -INFINITY, lf = tid < nt ? sq_log_sigmoid(sq_capped(pf, cap)) : 0.f;
+            float before = 0.f, after = 0.f;
+#pragma unroll
+            for (int t = 0; t < SQ_TC; t++) {
+                const float it = __shfl(li, t, 64), ft = __shfl(lf, t, 64), mn = fmaxf(ft + mrun, it);
+                if (tid == t) { before = ft + mrun; after = mn; }
+                mrun = mn;
+            }
+            if (tid < SQ_TC) {
+                gs[tid] = expf(before - after);
+                ds[tid] = expf(li - after);
+                if (last && tid < nt) mt[(long long)(t0 + tid) * H + h] = after;
+            }
+        }
+        float xv[NC][SQ_TC];
+#pragma unroll
+        for (int c = 0; c < NC; c++)
+#pragma unroll
+            for (int t = 0; t < SQ_TC; t++) xv[c][t] = pv[c][t];
+        __syncthreads();
+        if (t0 + SQ_TC < T) fetch(t0 + SQ_TC);
+#pragma unroll
+        for (int t = 0; t < SQ_TC; t++) {
+            const sq_f4 *ct = (const sq_f4 *)(cs + t * dp + s * SQ_NR), *bt = (const sq_f4 *)(bs + t * dp + s * SQ_NR);
+            const float g = gs[t], w = ds[t];
+            float u[NC], pp[NC][4];
+#pragma unroll
+            for (int c = 0; c < NC; c++) {
+                u[c] = w * xv[c][t];
+#pragma unroll
+                for (int e = 0; e < 4; e++) pp[c][e] = 0.f;
+            }
+#pragma unroll
+            for (int m4 = 0; m4 < SQ_NR / 4; m4++) {
+                const sq_f4 c4 = ct[m4], b4 = bt[m4];
+#pragma unroll
+                for (int c = 0; c < NC; c++)
+#pragma unroll
+                    for (int e = 0; e < 4; e++) {
+                        S[c][4 * m4 + e] = fmaf(g, S[c][4 * m4 + e], b4[e] * u[c]);
+                        pp[c][e] = fmaf(c4[e], S[c][4 * m4 + e], pp[c][e]);
+                    }
+            }
+#pragma unroll
+            for (int c = 0; c < NC; c++) {
+                const float p = sq_col_sum((pp[c][0] + pp[c][1]) + (pp[c][2] + pp[c][3]), R);
+                const int j = j0 + c * cpb;
+                if (s != 0 || t >= nt) continue;
+                if (j < P) o[(long long)(t0 + t) * ldo + vb + j] = p;
+                else if (j == P) nq[(long long)(t0 + t) * H + h] = p;
+            }
+        }
+    }
+#pragma unroll
+    for (int c = 0; c < NC; c++) {
+        const int j = j0 + c * cpb;
+        float *Sj = S0 + (long long)j * N + s * SQ_NR;
+        if (vec) {
+            if (j <= P && s * SQ_NR < N) {
+#pragma unroll
+                for (int m4 = 0; m4 < SQ_NR / 4; m4++) *(sq_f4 *)(Sj + 4 * m4) = sq_f4{S[c][4 * m4], S[c][4 * m4 + 1], S[c][4 * m4 + 2], S[c][4 * m4 + 3]};
+            }
+        } else {
+#pragma unroll
+            for (int m = 0; m < SQ_NR; m++)
+                if (j <= P && s * SQ_NR + m < N) Sj[m] = S[c][m];
+        }
+    }
+}
+void psk_mlstm_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, int64_t m_off, const float *q, const float *k, const float *v, int64_t ld, const float *iraw,
+                    const float *fraw, int64_t ldb, float cap, int H, int d, int dv, int T, float *o, int64_t ldo, float *nq, float *mt) {
+    const int R = sq_lanes_per_col(d), cpb = 256 / R;
+    const size_t lds = (size_t)(2 * SQ_TC * SQ_NR * R + 2 * SQ_TC) * 4;
+    const bool two = T > SQ_TC && dv > cpb;
+    const auto kernel = two ? sq_mlstm_scan_kernel<2> : sq_mlstm_scan_kernel<1>;
+    const int cols = two ? 2 * cpb : cpb;
+    hipLaunchKernelGGL(kernel, dim3((dv + cols) / cols, H), dim3(256), lds, st, step, (long long)state_off, (long long)m_off, q, k, v, (long long)ld, iraw, fraw, (long long)ldb, cap,
+                       1.f / sqrtf((float)d), H, d, dv, R, T, o, (long long)ldo, nq, mt);
+}
+// block (token, head), one wave
+__global__ __launch_bounds__(64) void sq_mlstm_finish_kernel(const ps_seq_step *step, long long m_off, float *o, long long ldo, const float *nq, const float *mt, const float *g,
+                                                             long long ldg, const float *w, float eps, int H, int dv) {
+    const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+    float *oh = o + (long long)t * ldo + (long long)h * dv;
+    const float *gh = g + (long long)t * ldg + (long long)h * dv, *wh = w + (long long)h * dv;
+    const float m = mt[(long long)t * H + h], den = fmaxf(fabsf(nq[(long long)t * H + h]), expf(-m)) + 1e-6f;
+    float s = 0.f;
+    for (int j = lane; j < dv; j += 64) { const float v = oh[j] / den; s += v * v; }
+#pragma unroll
+    for (int x = 32; x > 0; x >>= 1) s += __shfl_xor(s, x, 64);
+    const float inv = 1.f / sqrtf(s / (float)dv + eps);
+    for (int j = lane; j < dv; j += 64) oh[j] = oh[j] / den * inv * wh[j] * (1.f / (1.f + expf(-gh[j])));
+    if (t == (int)gridDim.x - 1 && lane == 0) step->state[m_off + h] = m;
+}
+void psk_mlstm_finish(hipStream_t st, const ps_seq_step *step, int64_t m_off, float *o, int64_t ldo, const float *nq, const float *mt, const float *g, int64_t ldg, const float *w,
+                      float eps, int H, int dv, int T) {
+    hipLaunchKernelGGL(sq_mlstm_finish_kernel, dim3(T, H), dim3(64), 0, st, step, (long long)m_off, o, (long long)ldo, nq, mt, g, (long long)ldg, w, eps, H, dv);
 }
 
 // o <- o silu(z), then each of gridDim.y equal parts (n numbers) divided by its own root mean square, times w: block (token, part); a thread re-reads only what it wrote

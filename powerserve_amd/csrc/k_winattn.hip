@@ -42,7 +42,7 @@ static __device__ __forceinline__ long long wa_front(long long p, int window, in
 __global__ __launch_bounds__(256) void winattn_prep_kernel(const ps_seq_step *step, long long ring_off, int cap, long long store_off, int pool, int keep, const float *y,
                                                            long long ldy, const float *qnorm, const float *knorm, float eps, int H, int G, int d, int dv, int rot_dims,
                                                            int pairing, const float *freq, float *qo, long long ldq, float qt_coef, int qt_every, int head_norm,
-                                                           int v_unit) {
+                                                           int v_unit, float rot_mag) {
     extern __shared__ float cs[];
     __shared__ float red[8];
     const int t = blockIdx.x, tid = threadIdx.x;
@@ -54,8 +54,8 @@ __global__ __launch_bounds__(256) void winattn_prep_kernel(const ps_seq_step *st
     const float qtemp = qt_every > 0 ? 1.f + qt_coef * logf((float)((pos + 1) / qt_every) + 1.f) : 1.f;
     for (int i = tid; i < half; i += 256) {
         const float ang = (float)pos * freq[i];
-        cs[i] = cosf(ang);
-        cs[half + i] = sinf(ang);
+        cs[i] = cosf(ang) * rot_mag;
+        cs[half + i] = sinf(ang) * rot_mag;
     }
     float a = 0.f, b = 0.f;
     if (qnorm && !head_norm) for (int i = tid; i < nq; i += 256) a += qt[i] * qt[i];
@@ -143,12 +143,12 @@ __global__ __launch_bounds__(256) void winattn_pool_kernel(const ps_seq_step *st
 
 void psk_winattn_prep(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, psk_front_store fs, const float *y, int64_t ldy, const float *qnorm,
                       const float *knorm, float eps, int H, int G, int d, int dv, int rot_dims, int pairing, const float *freq, int T, float *q, int64_t ldq, float qt_coef,
-                      int qt_every, int head_norm, int v_unit) {
+                      int qt_every, int head_norm, int v_unit, float rot_mag) {
     const int total = H * d + G * (d + dv);
     // few tokens: a token's elements over several blocks; with statistics per head, its heads (four per block)
     const int split = head_norm || v_unit ? (T >= 64 ? std::min(2, (H + 2 * G + 3) / 4) : std::min(32, (H + 2 * G + 3) / 4)) : T >= 64 ? 1 : std::min(16, (total + 511) / 512);
     hipLaunchKernelGGL(winattn_prep_kernel, dim3(T, split), dim3(256), (size_t)(rot_dims + 2) * 4, st, step, (long long)ring_off, cap, (long long)fs.off, fs.pool, fs.keep, y,
-                       (long long)ldy, qnorm, knorm, eps, H, G, d, dv, rot_dims, pairing, freq, q, (long long)ldq, qt_coef, qt_every, head_norm, v_unit);
+                       (long long)ldy, qnorm, knorm, eps, H, G, d, dv, rot_dims, pairing, freq, q, (long long)ldq, qt_coef, qt_every, head_norm, v_unit, rot_mag);
     if (fs.pool > 0 && T > 1 && G > 0) {
         const int rs = G * (d + dv);
         hipLaunchKernelGGL(winattn_pool_kernel, dim3((rs + 255) / 256, (T - 1) / fs.pool + 2), dim3(256), 0, st, step, (long long)ring_off, cap, (long long)fs.off, fs.pool, rs);

@@ -25,7 +25,8 @@ enum { PSD_ACT_NONE = 0, PSD_ACT_XIELU = 1, PSD_ACT_TANH = 2,
        PSD_ACT_SILU_PAIR = 3,   // rows 2i / 2i + 1 of W are a gate and its partner: out[t][i] = silu(row 2i) * (row 2i + 1), N / 2 outputs (bias: one per row, added first)
        PSD_ACT_RELU_PAIR = 4,   // the same with relu on the gate
        PSD_ACT_RELU2 = 5,       // max(z, 0)^2
-       PSD_ACT_SOFTCAP = 6 };   // act_p tanh(z / act_p)
+       PSD_ACT_SOFTCAP = 6,     // act_p tanh(z / act_p)
+       PSD_ACT_GELU_TANH = 7 }; // z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))
 
 // out[t][n] = alpha * act(sum_k A(t, k) W[n][k] + bias[n]),  t < T
 //   A(t, k) = a[row(t)][k], row(t) = t, or (a_row0 + t) mod a_mod when a_mod > 0 (rows of a ring), or, where a_step is given, rows of the
@@ -61,6 +62,12 @@ struct psk_dense_args {
     // g_ident_w[slot] * g_ident[row][n] to output n of its row instead of a product (g_ident NULL: nothing)
     const float *g_ident = nullptr, *g_ident_w = nullptr;
     int64_t g_ident_ld = 0;
+    // a factor from a second table (products that are not grouped, no paired activation): output n of row t is multiplied by em_table[token(t)][em_col + n] behind the activation;
+    // token(t) = em_tokens[t], or (em_tokens NULL) em_step->token0
+    const ps_dense *em_table = nullptr;
+    int64_t em_col = 0;
+    const int32_t *em_tokens = nullptr;
+    const ps_seq_step *em_step = nullptr;
 };
 int psk_dense(hipStream_t st, const psk_dense_args &a);
 void psk_dense_widen(hipStream_t st, const uint16_t *bf16, int64_t n, float *out);
@@ -83,7 +90,12 @@ void psk_norm_residual(hipStream_t st, float *x, const float *y, const float *w,
 // the norm taken over `groups` parts -- two norms of one vector share their statistics.  w1 / w2 NULL: that output is not made.
 void psk_front(hipStream_t st, const float *src, int64_t stride, int nmix, const float *mix, const int32_t *idx, float *xout, const float *w1, float *h, const float *w2,
                float *h2, int groups, float offset, float eps, int64_t n, int rows,
-               int center = 0); // 1: layer norms -- (x - mean) / sqrt(mean((x - mean)^2) + eps) over each part
+               int center = 0,  // 1: layer norms -- (x - mean) / sqrt(mean((x - mean)^2) + eps) over each part
+               const float *bias = nullptr); // added to h behind its weight
+// What a post-norm sublayer adds:  x[r] += norm(v) (offset + w) + bias, a layer norm (center) or an RMS norm over the whole row, bias may be NULL;  v = y[r], or, with the outputs of two
+// mixers side by side (w1 given; y2 NULL: one alone),  v = s1 rms(y[r]) w1 + s2 rms(y2[r]) w2 -- one launch from the output projections to the residual stream.
+void psk_postnorm(hipStream_t st, float *x, const float *y, const float *w1, float s1, const float *y2, const float *w2, float s2, const float *w, const float *bias, float offset,
+                  int center, float eps, int64_t n, int rows);
 // Element-wise gated recurrence.  y[t] = [ z | u | g ] (C each): S <- (1 - sigmoid(z)) S + sigmoid(z) c(u), c(u) = sigmoid(u) for negative u, else u + 0.5;
 // o[t] = S silu(g).  State [C] fp32 at step->state + state_off.
 void psk_mingru_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, const float *y, int64_t ldy, int64_t C, int T, float *o, int64_t ldo);
@@ -121,6 +133,15 @@ void psk_ssd_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, co
 void psk_gate_partnorm(hipStream_t st, float *o, int64_t ldo, const float *z, int64_t ldz, const float *w, int parts, float eps, int64_t n, int T);
 // o[t][h][:] = o / sqrt(mean_j o^2 + eps) * w(h, :) * silu(g[t][h][:]);  w_stride = dv (a weight per head) or 0 (one shared by the heads)
 void psk_headnorm_gate(hipStream_t st, float *o, int64_t ldo, const float *g, int64_t ldg, const float *w, int w_stride, float eps, int H, int dv, int T);
+// Matrix memory with exponential gates.  q, k [T][H*d], v [T][H*dv] (row stride ld), iraw / fraw [T][H] (row stride ldb) the gates' pre-activations; state per head [dv + 1][d] fp32 at
+// step->state + state_off (a column's d numbers together; the last column is n, the memory of k alone), the running maximum [H] at step->state + m_off.
+//   i = c(iraw), f = ln sigmoid(c(fraw)), c(z) = cap tanh(z / cap);  m' = max(f + m, i);  S <- exp(f + m - m') S + exp(i - m') k v^T, n alike
+// -> o[t][h] = S^T (q d^-1/2), nq[t][h] = n . (q d^-1/2), mt[t][h] = m'.  The maximum in the state is only read here: psk_mlstm_finish, behind every reader, writes it.
+void psk_mlstm_scan(hipStream_t st, const ps_seq_step *step, int64_t state_off, int64_t m_off, const float *q, const float *k, const float *v, int64_t ld, const float *iraw,
+                    const float *fraw, int64_t ldb, float cap, int H, int d, int dv, int T, float *o, int64_t ldo, float *nq, float *mt);
+// o[t][h] <- o / (max(|nq|, exp(-m)) + 1e-6), divided by its root mean square, times w [H dv], times sigmoid(g[t]); the last token's m goes to the state
+void psk_mlstm_finish(hipStream_t st, const ps_seq_step *step, int64_t m_off, float *o, int64_t ldo, const float *nq, const float *mt, const float *g, int64_t ldg, const float *w,
+                      float eps, int H, int dv, int T);
 
 // ---- k_ssd.hip
 // psk_ssd_scan for a portion, in chunks of 64 tokens on the fp32 matrix cores (same arguments; the same result up to rounding); _ok: the sizes it takes.
@@ -128,13 +149,20 @@ bool psk_ssd_chunked_ok(int N, int P);
 size_t psk_ssd_chunked_scratch(int H, int N, int P, int T);
 void psk_ssd_chunked(hipStream_t st, const ps_seq_step *step, int64_t state_off, const float *x, const float *B, const float *C, int64_t ld, const float *dtraw, int64_t ldb,
                      const float *a_log, const float *dt_bias, const float *skip, int H, int G, int N, int P, int T, float *scratch, float *o, int64_t ldo);
+// psk_mlstm_scan for a portion, in the same chunks (q, k, v 16-byte aligned, ld a multiple of 4; _ok: the sizes it takes)
+bool psk_mlstm_chunked_ok(int d, int dv);
+size_t psk_mlstm_chunked_scratch(int H, int d, int dv, int T);
+void psk_mlstm_chunked(hipStream_t st, const ps_seq_step *step, int64_t state_off, int64_t m_off, const float *q, const float *k, const float *v, int64_t ld, const float *iraw,
+                       const float *fraw, int64_t ldb, float cap, int H, int d, int dv, int T, float *scratch, float *o, int64_t ldo, float *nq, float *mt);
 
 // ---- k_moe.hip
 // Router of a mixture of experts, fp32: scores = sigmoid(router h[t]), or (softmax) the soft-max over all `experts` rows; choice scores = scores + correction (NULL: none);
 // with n_groups > 0 only rows of the `keep` groups (equal runs of neighbours) with the largest best choice score stay in the race; the `top` largest choice scores
 // (ties: the lower index) -> sel[t top + i], wgt[t top + i] (their SCORES, divided by their sum where norm_top, times scale); sgate[t] = sigmoid(shared_gate . h[t]) where given.
+// bias (NULL: none) joins the logits.  softmax 2: the logits themselves are the scores of the choice, and the weights are the soft-max over the chosen logits alone, times scale.
 void psk_moe_route(hipStream_t st, const float *h, int64_t ldh, const float *router, const float *shared_gate, int experts, int top, int norm_top, int64_t K, int T,
-                   int32_t *sel, float *wgt, float *sgate, int softmax = 0, const float *correction = nullptr, int n_groups = 0, int keep = 0, float scale = 1.f);
+                   int32_t *sel, float *wgt, float *sgate, int softmax = 0, const float *correction = nullptr, int n_groups = 0, int keep = 0, float scale = 1.f,
+                   const float *bias = nullptr);
 // The S slots sorted by expert: seg [experts + 1] (slots of expert e are list[seg[e] .. seg[e + 1])), list [S]
 void psk_moe_plan(hipStream_t st, const int32_t *sel, int S, int experts, int32_t *seg, int32_t *list);
 // x[t] += alpha * sum_i (y[t top + i], or, for a slot whose sel >= n_real (an identity expert), wgt[slot] * h[t]);  y NULL: only the identity slots; sel NULL: only y; store: x[t] = instead of +=
@@ -180,7 +208,8 @@ void psk_winattn_prep(hipStream_t st, const ps_seq_step *step, int64_t ring_off,
                       const float *knorm, float eps, int H, int G, int d, int dv, int rot_dims, int pairing, const float *freq, int T, float *q, int64_t ldq,
                       float qt_coef = 0.f, int qt_every = 0, // qt_every > 0: q[t] times 1 + qt_coef ln(floor((pos + 1) / qt_every) + 1)
                       int head_norm = 0, // 1: qnorm / knorm are [d] and the norms are taken per head
-                      int v_unit = 0);   // 1: every head's value divided by its own root mean square
+                      int v_unit = 0,    // 1: every head's value divided by its own root mean square
+                       float rot_mag = 1.f); // cos and sin are both multiplied by this
 // o[t][h] = gate(t, h) * soft-max attention of q[t][h] over the visible front store and the window's ring rows, scores times scale * temp[h], exp(sink[h]) in the
 // denominator; gate [T][..] raw (sigmoid here; column h, row stride ldg), temp / sink / gate may be NULL.
 void psk_winattn(hipStream_t st, const ps_seq_step *step, int64_t ring_off, int cap, psk_front_store fs, const float *q, int64_t ldq, const float *gate,

@@ -6,7 +6,7 @@
 // (their outputs are added, each times its scale), and a stretch of layers may run several times in a row with the same weights: the
 // unit that owns state is the layer RUN.  What a sequence carries: per run the tails of the input convolutions, and per mixer kind a
 // token-shift row + the wkv state, the short convolutions' tail + the delta-rule state, the gated-linear-attention state, the element-wise
-// recurrence's state, the ring of latents, or the ring of keys and values + the block means -- one fp32 block per slot, rings and means last,
+// recurrence's state, the matrix memory + its running maximum, the ring of latents, or the ring of keys and values + the block means -- one fp32 block per slot, rings and means last,
 // the rest zeroed when the slot is handed out.
 // A parallel layer may go without the input filter, take its two sublayers' inputs from two norms of the same vector, scale the sublayers' sum, and
 // hand on a weighted average of ALL earlier layers' results instead of its own (depth_mix): the results X_0 .. X_runs of a portion then live side by
@@ -14,7 +14,9 @@
 // The feed-forward may be a mixture of experts: the router (fp32) picks per token, the experts' products are grouped launches of the dense kernels.
 // A PRE-NORM layer is  x += mixer(norm1(x)); x += ff(norm2(x)):  no filter, nothing normed behind a sublayer, the second norm reads what the mixer left; its norms
 // (and the final one) may be layer norms (norm_center).
-// A POST-NORM layer is  x += norm1b(mixer(x)); x += norm2b(ff(x)):  the sublayers read the residual stream itself and only what they put out is normed.
+// A POST-NORM layer is  x += norm1b(mixer(x)); x += norm2b(ff(x)):  the sublayers read the residual stream itself and only what they put out is normed (layer norms with a bias,
+// possibly; the outputs of two mixers side by side may be normed one by one before they are summed).  Behind it a layer may add something for the token itself: its stretch of a second
+// embedding row, gated by the stream, through a projection and a norm of its own.
 // Attention layers may share keys and values: a layer with kv_from appends nothing and reads the ring (and the first tokens' rows) of the layer it names, which is sized for
 // the widest of its readers.  With a bigram embedding the last token of a portion is part of the slot's state.
 #include "ps_seq.h"
@@ -30,14 +32,14 @@ namespace {
 struct LayerPlan { // one layer RUN (and, as `side`, the second mixer of one)
     ps_seq_layer d;
     int layer = 0; // index into the descriptor's layers (runs of a looped layer share it, and its weights)
-    int64_t off_canon1 = 0, off_canon2 = 0, off_shift = 0, off_conv = 0, off_S = 0, off_ring = 0, off_pool = 0;
+    int64_t off_canon1 = 0, off_canon2 = 0, off_shift = 0, off_conv = 0, off_S = 0, off_m = 0, off_ring = 0, off_pool = 0;
     int cap = 0;          // latent / windowed attention: ring rows
     int64_t pool_rows = 0; // windowed attention: rows of the front store (block means, or the sequence's first tokens)
     int32_t keep_rows = 0; // of these, first tokens the append writes
     int owner = -1;        // windowed attention: the run whose ring and front store this one reads (-1: its own)
     float *freq = nullptr; // rot_dims / 2 angular frequencies (shared by the runs of a layer)
     float act_p = 0.f, act_q = 0.f;
-    float rot_mag = 1.f; // latent: the factor on cos and sin that comes with frequency scaling by wavelength
+    float rot_mag = 1.f; // attention: the factor on cos and sin that comes with frequency scaling by wavelength
     int64_t ncat = 0, cqkv = 0;
     // two mixers side by side whose first step is one stacked projection of the same input: the rows of both are ONE matrix (joint, with joint_bias), its
     // result has in_ld columns and this mixer's part starts at column in_off (in_ld == 0: the mixer multiplies by its own in_cat)
@@ -67,7 +69,9 @@ struct ps_hip_seq {
     int32_t *moe_sel = nullptr, *moe_seg = nullptr, *moe_list = nullptr; // mixture of experts: expert per slot, the slots sorted by expert
     float *moe_wgt = nullptr, *moe_sg = nullptr, *moe_y = nullptr;       // weight per slot, the shared expert's gate per token, per-slot results (top > 1)
     float *win_scratch = nullptr; // the windowed attention's single-token partials
-    float *ssd_scratch = nullptr; // the chunked state-space recurrence: a state per chunk
+    float *ssd_scratch = nullptr; // the chunked recurrences: a state per chunk (and the matrix memory's gates)
+    float *lstm_aux = nullptr;    // matrix memory: [max_batch][heads] products with n, then as many running maxima
+    int64_t lstm_aux_n = 0;
     float *abs_scratch = nullptr; // the absorbed single-token attention's folded queries, attended latents and per-tile partials
     void *pack = nullptr; // the wide mat-mul's bfloat16 operand copy
     size_t pack_bytes = 0;
@@ -100,7 +104,7 @@ __global__ void seq_advance_kernel(ps_seq_step *s, const int32_t *amax, int32_t 
     s->pos0 += 1;
 }
 
-static const int SSD_CHUNKED_FROM = 32; // tokens from which a portion's state-space recurrence runs in chunks (fewer: the scan)
+static const int SSD_CHUNKED_FROM = 32; // tokens from which a portion's state-space recurrence or matrix memory runs in chunks (fewer: the scan)
 
 static int seq_fail(ps_hip_ctx *c, const std::string &msg) { c->err = msg; return 2; }
 
@@ -134,6 +138,7 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
             return fail("bigram multipliers");
         m->off_prev = off; off += 4;
     }
+    if (desc->side_embed && (desc->side_dim <= 0 || !shape(desc->side_embed, desc->vocab, (int64_t)desc->n_layers * desc->side_dim))) return fail("side_embed shape");
     bool depth = false;
     std::vector<int> order; // layer index of every run
     {
@@ -207,6 +212,9 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
             if (G <= 0 || H % G || dv <= 0 || dv > 256 || l.rot_dims < 0 || l.rot_dims > d || (l.rot_dims & 1) || l.window < 0 || l.pool < 0)
                 return at + "windowed attention sizes (heads a multiple of kv_heads, vdim <= 256, even rot_dims <= dim)";
             if (l.rot_pairing != PS_ROT_HALVES && l.rot_pairing != PS_ROT_NEIGHBOURS) return at + "rot_pairing";
+            if (l.yarn_factor != 0.f && (!(l.yarn_factor > 0.f) || l.yarn_original <= 0 || !(l.yarn_fast > 0.f) || !(l.yarn_slow > 0.f) || !(l.rot_base > 1.f)))
+                return at + "windowed attention: frequency scaling constants";
+            P.rot_mag = l.yarn_factor > 0.f ? (float)(0.1 * log((double)l.yarn_factor) + 1.0) : 1.f;
             if (l.gated < 0 || l.gated > 2) return at + "gated: 0 (none), 1 (a row per head) or 2 (a row per output element)";
             if (l.keep_first < 0 || (l.pool > 0 && (l.keep_first > 0 || l.dist_slope))) return at + "first tokens and distance slopes are not built together with pooled blocks";
             if (l.kv_from < 0 || (l.kv_from > 0 && (desc->loop_times > 1 || l.kv_from > P.layer || l.pool > 0))) return at + "kv_from names an earlier layer (no loop, no pooled blocks)";
@@ -247,6 +255,18 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
             n2 = std::max(n2, P.cqkv);
             n3 = std::max(n3, inner);
             m->weight_bytes += dense_bytes(l.in_cat) + dense_bytes(l.out);
+        } else if (l.kind == PS_MIX_MLSTM) {
+            if (d > 256) return at + "matrix memory: dim > 256 is not supported by the scan kernel";
+            if (dv <= 0 || l.gate_cap < 0.f) return at + "matrix memory sizes";
+            P.ncat = 2 * H * d + 2 * H * dv + 2 * H;
+            if (!shape(l.in_cat, P.ncat, W) || !shape(l.out, W, H * dv) || !l.onorm) return at + "matrix memory tensors";
+            P.off_m = off; off += H;
+            off = (off + 3) / 4 * 4; // (16-byte pieces of the state)
+            P.off_S = off; off += H * (dv + 1) * d;
+            n1 = std::max(n1, P.ncat);
+            n3 = std::max(n3, H * dv);
+            m->lstm_aux_n = std::max(m->lstm_aux_n, B * H);
+            m->weight_bytes += dense_bytes(l.in_cat) + dense_bytes(l.out);
         } else if (l.kind == PS_MIX_MINGRU) {
             P.ncat = 3 * d;
             if (!shape(l.in_cat, P.ncat, W) || !shape(l.out, W, d)) return at + "gated recurrence tensors";
@@ -270,7 +290,15 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
         if (l.form == PS_LAYER_POSTNORM && (l.norm1 || l.norm2 || l.canon1 || l.canon2 || l.depth_mix)) return fail(at + "a post-norm layer has no norm in front of a sublayer, no input filter and no depth average");
         if (l.form == PS_LAYER_POSTNORM && (!l.norm1b || (l.ff_kind != PS_FF_NONE && !l.norm2b))) return fail(at + "output norm missing");
         if (l.form == PS_LAYER_PRENORM && (l.canon1 || l.canon2 || l.norm1b || l.norm2b || l.depth_mix)) return fail(at + "a pre-norm layer has no input filter, no norm behind a sublayer and no depth average");
-        if (l.form != PS_LAYER_PRENORM && desc->norm_center) return fail(at + "layer norms (norm_center) are built for pre-norm layers");
+        if (l.form != PS_LAYER_PRENORM && l.form != PS_LAYER_POSTNORM && desc->norm_center) return fail(at + "layer norms (norm_center) are built for pre-norm and post-norm layers");
+        if (l.form != PS_LAYER_POSTNORM && (l.norm1b_bias || l.norm2b_bias || l.mix_onorm || l.side_gate)) return fail(at + "norm biases, norms of a mixer's own output and a token input are built for post-norm layers");
+        if (l.form == PS_LAYER_POSTNORM && m->groups > 1 && (desc->norm_center || l.norm1b_bias || l.norm2b_bias || l.mix_onorm)) return fail(at + "layer norms, norm biases and mix_onorm of a post-norm layer take the whole row");
+        if (l.beside && !l.mix_onorm != !l.beside->mix_onorm) return fail(at + "mix_onorm: both of two mixers side by side, or none");
+        if (l.side_gate || l.side_proj || l.side_norm) {
+            if (!desc->side_embed || !shape(l.side_gate, desc->side_dim, W) || !shape(l.side_proj, W, desc->side_dim) || !l.side_norm) return fail(at + "token input tensors");
+            n4 = std::max<int64_t>(n4, desc->side_dim);
+            m->weight_bytes += dense_bytes(l.side_gate) + dense_bytes(l.side_proj);
+        }
         if ((!l.norm1 && l.form != PS_LAYER_POSTNORM) || (l.form == PS_LAYER_SEQUENTIAL && !l.norm1b) || (l.form == PS_LAYER_SEQUENTIAL && !l.canon1)) return fail(at + "norm / canon missing");
         if (l.canon1) { P.off_canon1 = off; off += (int64_t)(desc->canon_taps - 1) * W; }
         if (l.canon1 && (l.norm2 && l.form == PS_LAYER_PARALLEL)) return fail(at + "a parallel layer with an input filter has one norm");
@@ -372,14 +400,14 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
         const double factor = win && P.d.rot_factor != 0.f ? (double)P.d.rot_factor : 1.0;
         std::vector<float> f(half);
         for (int i = 0; i < half; i++) f[i] = (float)(pow((double)P.d.rot_base, -2.0 * i / (double)P.d.rot_dims) / factor);
-        if (lat && P.d.yarn_factor > 0.f) {
+        if (P.d.yarn_factor > 0.f) {
             // frequency scaling by wavelength: pairs that turn often within the original context keep their frequency, slow ones are divided by the factor, a ramp between
             const double dims = P.d.rot_dims, base = P.d.rot_base, pi = 3.14159265358979323846;
             auto turn_index = [&](double turns) { return dims * log((double)P.d.yarn_original / (2.0 * pi * turns)) / (2.0 * log(base)); };
             const double lo = std::max(floor(turn_index(P.d.yarn_fast)), 0.0), hi = std::min(ceil(turn_index(P.d.yarn_slow)), dims - 1.0);
             for (int i = 0; i < half; i++) {
                 const double fi = pow(base, -2.0 * i / dims), ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
-                f[i] = (float)(fi / (double)P.d.yarn_factor * ramp + fi * (1.0 - ramp));
+                f[i] = (float)((fi / (double)P.d.yarn_factor * ramp + fi * (1.0 - ramp)) / factor);
             }
         }
         ok = ok && alloc((void **)&P.freq, half * 4);
@@ -388,34 +416,37 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
     });
     {
         // the stacked input projections of two mixers side by side, joined once per layer (its runs share the copy)
-        auto stacked = [](int kind) { return kind == PS_MIX_WINATTN || kind == PS_MIX_GLA || kind == PS_MIX_DELTA || kind == PS_MIX_MINGRU; };
+        auto stacked = [](int kind) { return kind == PS_MIX_WINATTN || kind == PS_MIX_GLA || kind == PS_MIX_DELTA || kind == PS_MIX_MINGRU || kind == PS_MIX_MLSTM; };
         std::map<int, std::pair<const ps_dense *, const float *>> joint_of;
         for (auto &P : m->L) {
             if (!ok || !P.side || !stacked(P.d.kind) || !stacked(P.side->d.kind) || P.d.in_cat->dtype != P.side->d.in_cat->dtype) continue;
             const ps_dense *a = P.d.in_cat, *b = P.side->d.in_cat;
+            const int64_t skip = (a->N + 3) / 4 * 4 - a->N; // (rows of zeros between them: the second mixer's columns start 16-byte aligned)
             auto it = joint_of.find(P.layer);
             if (it == joint_of.end()) {
-                const size_t es = a->dtype == PS_BF16 ? 2 : 4, na = (size_t)a->N * a->K * es, nb = (size_t)b->N * b->K * es;
+                const size_t es = a->dtype == PS_BF16 ? 2 : 4, na = (size_t)a->N * a->K * es, nb = (size_t)b->N * b->K * es, nz = (size_t)skip * a->K * es;
                 auto j = new ps_dense();
                 m->joints.push_back(j);
-                j->dtype = a->dtype; j->N = a->N + b->N; j->K = a->K;
-                ok = ok && alloc(&j->data, na + nb) && hipMemcpyAsync(j->data, a->data, na, hipMemcpyDeviceToDevice, c->stream) == hipSuccess &&
-                     hipMemcpyAsync((char *)j->data + na, b->data, nb, hipMemcpyDeviceToDevice, c->stream) == hipSuccess;
+                j->dtype = a->dtype; j->N = a->N + skip + b->N; j->K = a->K;
+                ok = ok && alloc(&j->data, na + nz + nb);
+                if (ok) psk_fill(c->stream, (float *)j->data, 0.f, (int64_t)((na + nz) / 4));
+                ok = ok && hipMemcpyAsync(j->data, a->data, na, hipMemcpyDeviceToDevice, c->stream) == hipSuccess &&
+                     hipMemcpyAsync((char *)j->data + na + nz, b->data, nb, hipMemcpyDeviceToDevice, c->stream) == hipSuccess;
                 float *bias = nullptr;
                 if (ok && (P.d.in_bias || P.side->d.in_bias)) {
                     ok = alloc((void **)&bias, (size_t)j->N * 4);
                     if (ok) {
                         psk_fill(c->stream, bias, 0.f, j->N);
                         if (P.d.in_bias) ok = ok && hipMemcpyAsync(bias, P.d.in_bias, (size_t)a->N * 4, hipMemcpyDeviceToDevice, c->stream) == hipSuccess;
-                        if (P.side->d.in_bias) ok = ok && hipMemcpyAsync(bias + a->N, P.side->d.in_bias, (size_t)b->N * 4, hipMemcpyDeviceToDevice, c->stream) == hipSuccess;
+                        if (P.side->d.in_bias) ok = ok && hipMemcpyAsync(bias + a->N + skip, P.side->d.in_bias, (size_t)b->N * 4, hipMemcpyDeviceToDevice, c->stream) == hipSuccess;
                     }
                 }
                 ok = ok && hipStreamSynchronize(c->stream) == hipSuccess;
                 it = joint_of.emplace(P.layer, std::make_pair((const ps_dense *)j, (const float *)bias)).first;
             }
             P.joint = it->second.first; P.joint_bias = it->second.second;
-            P.in_ld = P.side->in_ld = a->N + b->N;
-            P.in_off = 0; P.side->in_off = a->N;
+            P.in_ld = P.side->in_ld = (a->N + skip + b->N + 3) / 4 * 4;
+            P.in_off = 0; P.side->in_off = a->N + skip;
             n1 = std::max(n1, P.in_ld);
         }
     }
@@ -443,12 +474,14 @@ int ps_hip_seq_create(ps_hip_ctx *c, const ps_seq_desc *desc, ps_hip_seq **out) 
         if (wb) ok = ok && alloc((void **)&m->win_scratch, wb);
         size_t sb = 0;
         mixers([&](LayerPlan &P) {
+            if (P.d.kind == PS_MIX_MLSTM && B >= SSD_CHUNKED_FROM && psk_mlstm_chunked_ok(P.d.dim, P.d.vdim)) sb = std::max(sb, psk_mlstm_chunked_scratch(P.d.heads, P.d.dim, P.d.vdim, (int)B));
             if (P.d.kind == PS_MIX_SSD && B >= SSD_CHUNKED_FROM && psk_ssd_chunked_ok(P.d.dim, P.d.vdim)) sb = std::max(sb, psk_ssd_chunked_scratch(P.d.heads, P.d.dim, P.d.vdim, (int)B));
         });
         if (sb) ok = ok && alloc((void **)&m->ssd_scratch, sb);
+        if (m->lstm_aux_n) ok = ok && alloc((void **)&m->lstm_aux, (size_t)m->lstm_aux_n * 2 * 4);
     }
     if (desc->compute == 0) { // the wide mat-mul's operand copy: the widest input of any matrix x a portion's rows, or the window's rows x the latent
-        int64_t kmax = W, kvrows = 0, kvk = 0;
+        int64_t kmax = std::max<int64_t>(W, desc->side_dim), kvrows = 0, kvk = 0;
         mixers([&](LayerPlan &P) {
             kmax = std::max<int64_t>({kmax, P.d.ff, P.d.shared_ff, P.d.heads * (int64_t)std::max(P.d.dim, P.d.vdim), P.d.q_rank, P.d.decay_rank});
             if (P.d.kind == PS_MIX_LATENT) { kvrows = std::max<int64_t>(kvrows, P.d.window - 1 + B); kvk = std::max<int64_t>(kvk, P.d.kv_rank); }
@@ -532,14 +565,14 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
             psk_causal_conv(st, m->step, tail_off, m->hn, W, cw, D.canon_taps, 0, W, T, m->h, W);
         }
     };
-    // One mixer on the input `in`.  Its output projection writes m->y (into == NULL) or adds out_scale times its result to `into`.
-    auto mixer = [&](const LayerPlan &P, const float *in, float *into, float out_scale) {
+    // One mixer on the input `in`.  Its output projection writes out_scale times its result to `store` (NULL: m->y), or (into given) adds it there.
+    auto mixer = [&](const LayerPlan &P, const float *in, float *into, float out_scale, float *store = nullptr) {
         const ps_seq_layer &l = P.d;
         const int64_t H = l.heads, d = l.dim, dv = l.vdim;
         float *t1 = m->t1 + P.in_off;                       // this mixer's columns of the (possibly joint) input projection
         const int64_t ld1 = P.in_ld ? P.in_ld : P.ncat;
         auto out_proj = [&](const float *a, int64_t lda) {
-            auto g = mm(l.out, a, lda, into ? into : m->y, W);
+            auto g = mm(l.out, a, lda, into ? into : store ? store : m->y, W);
             g.alpha = out_scale; g.accum = into ? 1 : 0; g.bias = l.out_bias;
             psk_dense(st, g);
         };
@@ -591,7 +624,8 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
             }
             const bool reads = P.owner >= 0; // (another layer's keys and values: queries only)
             psk_winattn_prep(st, m->step, P.off_ring, P.cap, psk_front_store{P.off_pool, l.pool, reads ? 0 : P.keep_rows}, t1, ld1, l.qnorm, l.knorm, D.norm_eps, (int)H,
-                             reads ? 0 : (int)G, (int)d, (int)dv, l.rot_dims, l.rot_pairing, P.freq, T, m->t2, Hd, l.qtemp_coef, l.qtemp_every, l.head_norm, l.v_unit);
+                             reads ? 0 : (int)G, (int)d, (int)dv, l.rot_dims, l.rot_pairing, P.freq, T, m->t2, Hd, l.qtemp_coef, l.qtemp_every, l.head_norm, l.v_unit,
+                             P.rot_mag);
             const psk_front_store fs{P.off_pool, l.pool, l.keep_first};
             const float *gate = l.gated ? t1 + Hd + (reads ? 0 : G * d + G * dv) : nullptr;
             const int ge = l.gated == 2; // a gate per output element
@@ -618,6 +652,22 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
                 psk_ssd_scan(st, m->step, P.off_S, x, Bv, Cv, P.cqkv, dt, ld1, l.a_log, l.dt_bias, l.skip, (int)H, l.kv_heads, (int)d, (int)dv, T, m->t3, inner);
             psk_gate_partnorm(st, m->t3, inner, t1, ld1, l.onorm, l.norm_parts, D.norm_eps, inner, T);
             out_proj(m->t3, inner);
+        } else if (l.kind == PS_MIX_MLSTM) {
+            // t1 = [ q | k | v | g | i | f ] (+ bias); the memory -> t3, its products with n and running maxima -> lstm_aux; denominator, head norm and gate; out
+            const int64_t Hd = H * d, Hv = H * dv;
+            if (!P.in_ld) {
+                auto g = mm(l.in_cat, in, W, t1, ld1);
+                g.bias = l.in_bias;
+                psk_dense(st, g);
+            }
+            const float *k = t1 + Hd, *v = k + Hd, *g = v + Hv, *iz = g + Hv, *fz = iz + H;
+            float *nq = m->lstm_aux, *mt = nq + m->lstm_aux_n;
+            if (T >= SSD_CHUNKED_FROM && !tiled && m->ssd_scratch && ld1 % 4 == 0 && psk_mlstm_chunked_ok((int)d, (int)dv))
+                psk_mlstm_chunked(st, m->step, P.off_S, P.off_m, t1, k, v, ld1, iz, fz, ld1, l.gate_cap, (int)H, (int)d, (int)dv, T, m->ssd_scratch, m->t3, Hv, nq, mt);
+            else
+                psk_mlstm_scan(st, m->step, P.off_S, P.off_m, t1, k, v, ld1, iz, fz, ld1, l.gate_cap, (int)H, (int)d, (int)dv, T, m->t3, Hv, nq, mt);
+            psk_mlstm_finish(st, m->step, P.off_m, m->t3, Hv, nq, mt, g, ld1, l.onorm, D.norm_eps, (int)H, (int)dv, T);
+            out_proj(m->t3, Hv);
         } else if (l.kind == PS_MIX_MINGRU) {
             // t1 = [ z | x | g ] (+ bias); the recurrence and the gate -> t3; out
             if (!P.in_ld) {
@@ -691,7 +741,7 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
         const int E = l.experts, rows = E + l.moe_identity, top = l.top, S = T * top;
         const int act = l.ff_kind == PS_FF_MOE_RELU2 ? PSD_ACT_RELU2 : PSD_ACT_SILU_PAIR;
         psk_moe_route(st, in, W, l.router, l.shared_gate, rows, top, l.moe_norm_top, W, T, m->moe_sel, m->moe_wgt, m->moe_sg, l.moe_softmax, l.moe_correction, l.moe_groups,
-                      l.moe_keep, l.moe_scale != 0.f ? l.moe_scale : 1.f);
+                      l.moe_keep, l.moe_scale != 0.f ? l.moe_scale : 1.f, l.router_bias);
         const bool mv = !tiled && T <= 8 && (size_t)std::max<int64_t>(W, (int64_t)top * l.ff) * 4 + 64 <= 128 * 1024;
         if (!mv) psk_moe_plan(st, m->moe_sel, S, rows, m->moe_seg, m->moe_list);
         auto grouped = [&](psk_dense_args &g) {
@@ -755,13 +805,33 @@ static void seq_layers(ps_hip_seq *m, float *state, int T, int64_t pos0, bool an
             }
         } else if (l.form == PS_LAYER_POSTNORM) {
             // x += norm_b(mixer(x)), then x += norm_b(ff(x)): a sublayer's first product reads the residual stream, its last one writes y
+            auto post = [&](const float *w, const float *b) {
+                if (D.norm_center || b) psk_postnorm(st, m->x, m->y, nullptr, 0.f, nullptr, nullptr, 0.f, w, b, D.norm_offset, D.norm_center, D.norm_eps, W, T);
+                else boundary(m->y, w, nullptr, nullptr, 0);
+            };
             joint_in(P, m->x);
-            mixer(P, m->x, nullptr, l.mix_scale);
-            if (P.side) mixer(*P.side, m->x, m->y, P.side->d.mix_scale);
-            boundary(m->y, l.norm1b, nullptr, nullptr, 0);
+            if (l.mix_onorm) { // the mixers' outputs side by side (y and h), normed one by one, summed, normed and added in one launch
+                mixer(P, m->x, nullptr, 1.f);
+                if (P.side) mixer(*P.side, m->x, nullptr, 1.f, m->h);
+                psk_postnorm(st, m->x, m->y, l.mix_onorm, l.mix_scale, P.side ? m->h : nullptr, P.side ? P.side->d.mix_onorm : nullptr, P.side ? P.side->d.mix_scale : 0.f, l.norm1b,
+                             l.norm1b_bias, D.norm_offset, D.norm_center, D.norm_eps, W, T);
+            } else {
+                mixer(P, m->x, nullptr, l.mix_scale);
+                if (P.side) mixer(*P.side, m->x, m->y, P.side->d.mix_scale);
+                post(l.norm1b, l.norm1b_bias);
+            }
             if (l.ff_kind != PS_FF_NONE) {
                 feed_forward(P, m->x, m->y, 1.f, true);
-                boundary(m->y, l.norm2b, nullptr, nullptr, 0);
+                post(l.norm2b, l.norm2b_bias);
+            }
+            if (l.side_gate) { // the token's own input to this layer: (gelu(gate x) * its stretch of the table row) in one product, the projection, norm and add
+                auto g = mm(l.side_gate, m->x, W, m->t4, D.side_dim);
+                g.act = PSD_ACT_GELU_TANH;
+                g.em_table = D.side_embed; g.em_col = (int64_t)P.layer * D.side_dim; g.em_tokens = from_step ? nullptr : m->tokens; g.em_step = m->step;
+                psk_dense(st, g);
+                psk_dense(st, mm(l.side_proj, m->t4, D.side_dim, m->y, W));
+                if (T == 1 && !tiled) psk_boundary1(st, m->step, m->x, m->y, l.side_norm, nullptr, nullptr, 1, 0, 0.f, D.norm_eps, W, nullptr, nullptr);
+                else psk_norm_residual(st, m->x, m->y, l.side_norm, 0.f, D.norm_eps, W, T);
             }
         } else if (l.form == PS_LAYER_PARALLEL && !l.canon1) {
             // No input filter: one launch makes the layer's input (with depth_mix: the previous layer's average over X_0 .. X_li, kept as this layer's X to add
@@ -812,9 +882,9 @@ static void seq_head(ps_hip_seq *m, const int32_t *idx, int rows) {
     if (m->hist) { // what the last layer hands on (its depth average, or its own result) and the final norm in one launch
         const int runs = (int)m->L.size();
         psk_front(st, m->hist, (int64_t)D.max_batch * D.width, runs + 1, m->L[runs - 1].d.depth_mix, idx, nullptr, D.final_norm, m->xn, nullptr, nullptr, m->groups,
-                  D.norm_offset, D.norm_eps, D.width, rows);
-    } else if (D.norm_center) {
-        psk_front(st, m->x, 0, 1, nullptr, idx, nullptr, D.final_norm, m->xn, nullptr, nullptr, m->groups, D.norm_offset, D.norm_eps, D.width, rows, 1);
+                  D.norm_offset, D.norm_eps, D.width, rows, 0, D.final_norm_bias);
+    } else if (D.norm_center || D.final_norm_bias) {
+        psk_front(st, m->x, 0, 1, nullptr, idx, nullptr, D.final_norm, m->xn, nullptr, nullptr, m->groups, D.norm_offset, D.norm_eps, D.width, rows, D.norm_center, D.final_norm_bias);
     } else {
         psk_rmsnorm(st, m->x, D.width, idx, D.final_norm, D.norm_offset, D.norm_eps, D.width, rows, m->xn, D.width, m->groups);
     }
@@ -944,7 +1014,7 @@ int ps_hip_seq_bench_kernel(ps_hip_seq *m, int which, int T, int reps, double *u
             for (int first = 0; first < (mv && P.d.moe_identity ? 64 : 1); first++) {
                 if (first && !embed_from(first)) return seq_fail(c, "seq_bench_kernel: embedding");
                 psk_moe_route(c->stream, m->h, W, P.d.router, P.d.shared_gate, rows, top, P.d.moe_norm_top, W, T, m->moe_sel, m->moe_wgt, m->moe_sg, P.d.moe_softmax,
-                              P.d.moe_correction, P.d.moe_groups, P.d.moe_keep, P.d.moe_scale != 0.f ? P.d.moe_scale : 1.f);
+                              P.d.moe_correction, P.d.moe_groups, P.d.moe_keep, P.d.moe_scale != 0.f ? P.d.moe_scale : 1.f, P.d.router_bias);
                 PS_CHECK(c, hipMemcpyAsync(sel.data(), m->moe_sel, (size_t)S * 4, hipMemcpyDeviceToHost, c->stream));
                 PS_CHECK(c, hipStreamSynchronize(c->stream));
                 bool all_real = true;

@@ -104,7 +104,8 @@ SeqLayer._fields_ = ([(n, C.c_int32) for n in ("kind", "heads", "kv_heads", "dim
                 [("ff_up_bias", C.c_void_p), ("ff_down_bias", C.c_void_p)] +
                 [(n, C.c_int32) for n in ("moe_identity", "moe_softmax", "moe_groups", "moe_keep", "moe_weight_output")] + [("moe_correction", C.c_void_p)] +
                 [("moe_scale", C.c_float), ("out_bias", C.c_void_p), ("dist_slope", C.c_void_p)] + [(n, C.c_int32) for n in ("keep_first", "kv_from", "norm_parts")] +
-                [("conv_bias", C.c_void_p), ("skip", C.c_void_p)])
+                [(n, C.c_void_p) for n in ("conv_bias", "skip", "norm1b_bias", "norm2b_bias", "mix_onorm", "router_bias", "side_gate", "side_proj", "side_norm")] +
+                [("gate_cap", C.c_float)])
 
 
 class SeqDesc(C.Structure):
@@ -113,7 +114,8 @@ class SeqDesc(C.Structure):
                 [("norm_eps", C.c_float), ("norm_offset", C.c_float), ("logit_scale", C.c_float)] +
                 [("embed", C.c_void_p), ("head", C.c_void_p), ("final_norm", C.c_void_p), ("layers", C.POINTER(SeqLayer))] +
                 [("embed_scale", C.c_float)] + [(n, C.c_int32) for n in ("loop_start", "loop_stop", "loop_times", "max_context", "norm_groups", "norm_center")] +
-                [("bigram", C.c_void_p)] + [(n, C.c_int64) for n in ("bigram_buckets", "bigram_mul_prev", "bigram_mul_cur")] + [("logit_softcap", C.c_float)])
+                [("bigram", C.c_void_p)] + [(n, C.c_int64) for n in ("bigram_buckets", "bigram_mul_prev", "bigram_mul_cur")] + [("logit_softcap", C.c_float), ("side_dim", C.c_int32)] +
+                [("side_embed", C.c_void_p), ("final_norm_bias", C.c_void_p)])
 
 
 _LIB = None

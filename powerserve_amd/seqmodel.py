@@ -44,6 +44,14 @@ scale on what they put out (loaded as one vector, weight times scale).  A hashed
                     head, biases on all four projections; with 'kv_from' a layer reads another one's cached keys and values
   latent_attention  as Pokatar's, with rotary on neighbouring pairs and plain frequencies
 Feed-forward: squared-relu experts behind a soft-max router in fp32, the chosen scores (not renormalised) times router.scale on the outputs, a shared expert.
+
+Sogavik: POST-NORM layers whose norms are layer norms with a weight and a bias,  x += ln1(mix(x)); x += ln2(mlp(x)),  then an input of the layer's own for the token itself:
+x += rms(proj (gelu(gate x) * e)) * norm  with e the layer's stretch ('token_side'.dim numbers) of a second embedding row.  Mixers:
+  attention         grouped-query attention over a sliding window: biases on q / k / v, RMS norms over the whole q / k projections, rotate-half rotary on the first rot.dims numbers of a
+                    head with frequencies scaled by wavelength, a sigmoid gate per head
+  parallel          two mixers side by side, half the sum of their outputs, each RMS-normed over the width first:
+                    left  = such an attention (no gate), right = a matrix memory with exponential gates under a running maximum (mLSTM), per-head norm and a sigmoid gate
+Feed-forward: SiLU-gated experts, the largest logits (with a bias, fp32) chosen, the soft-max over the chosen logits alone on their outputs.
 """
 from __future__ import annotations
 
@@ -56,7 +64,7 @@ import numpy as np
 from . import hip
 from .safetensors_io import SafeTensors
 
-MIX_WKV, MIX_DELTA, MIX_LATENT, MIX_WINATTN, MIX_GLA, MIX_MINGRU, MIX_SSD = 1, 2, 3, 4, 5, 6, 7
+MIX_WKV, MIX_DELTA, MIX_LATENT, MIX_WINATTN, MIX_GLA, MIX_MINGRU, MIX_SSD, MIX_MLSTM = 1, 2, 3, 4, 5, 6, 7, 8
 FF_NONE, FF_DENSE_XIELU, FF_DENSE_SWIGLU, FF_MOE_SWIGLU, FF_DENSE_RELU_GLU, FF_MOE_RELU2 = 0, 1, 2, 3, 4, 5
 LAYER_SEQUENTIAL, LAYER_PARALLEL, LAYER_PRENORM, LAYER_POSTNORM = 0, 1, 2, 3
 ROT_HALVES, ROT_NEIGHBOURS = 0, 1
@@ -133,9 +141,17 @@ def _stack(st: SafeTensors, names: list) -> np.ndarray:
     return np.concatenate([st.bf16_bits(n) for n in names], axis=0)
 
 
-def window_attention_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str):
+def wavelength_scaling(L, rot: dict):
+    """Rotary frequencies scaled by wavelength, where the configuration's rot has a 'scaling' (factor, original, fast, slow)."""
+    sc = rot.get("scaling") or {}
+    if sc:
+        L.yarn_factor, L.yarn_fast, L.yarn_slow, L.yarn_original = float(sc["factor"]), float(sc["fast"]), float(sc["slow"]), int(sc["original"])
+
+
+def window_attention_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str, pairing: int = ROT_NEIGHBOURS, by_wavelength: bool = False):
     """Fill descriptor L with a windowed-attention mixer (MIX_WINATTN) from the tensors under prefix m and its configuration mc.  Whatever the
-    configuration or the file does not have does not exist: no bias, no norm, no temperature, no sink, no gate, no rotation, no pooled blocks."""
+    configuration or the file does not have does not exist: no bias, no norm, no temperature, no sink, no gate, no rotation, no pooled blocks.
+    by_wavelength: rot.scaling scales the frequencies by wavelength (else all of them by its factor)."""
     L.kind = MIX_WINATTN
     L.heads, L.dim = int(mc["heads"]), int(mc["dim"])
     L.kv_heads, L.vdim = int(mc.get("kv_heads") or L.heads), int(mc.get("vdim") or L.dim)
@@ -143,8 +159,11 @@ def window_attention_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str)
         raise ConfigError(f"{where}: {L.heads} heads over {L.kv_heads} key / value heads")
     mask, rot = mc.get("mask") or {}, mc.get("rot") or {}
     L.window, L.pool = int(mask.get("size") or 0), int(mask.get("pool") or 0)
-    L.rot_dims, L.rot_base, L.rot_pairing = int(rot.get("dims") or 0), float(rot.get("base") or 10000.0), ROT_NEIGHBOURS
-    L.rot_factor = float((rot.get("scaling") or {}).get("factor") or 1.0)
+    L.rot_dims, L.rot_base, L.rot_pairing = int(rot.get("dims") or 0), float(rot.get("base") or 10000.0), pairing
+    if by_wavelength:
+        wavelength_scaling(L, rot)
+    else:
+        L.rot_factor = float((rot.get("scaling") or {}).get("factor") or 1.0)
     L.scale = float(mc["scale"]) if mc.get("scale") is not None else L.dim ** -0.5
     L.softcap = float(mc.get("softcap") or 0.0)
     qt = mc.get("q_temp") or {}
@@ -207,9 +226,10 @@ def _gate_up(st: SafeTensors, p: str, ff: int, width: int, where: str) -> np.nda
     return np.stack([gate, upw], axis=1).reshape(2 * ff, width)
 
 
-def gated_feed_forward(L, st: SafeTensors, up, p: str, mlp: dict, width: int, where: str):
+def gated_feed_forward(L, st: SafeTensors, up, p: str, mlp: dict, width: int, where: str, chosen_softmax: bool = False):
     """Fill descriptor L's feed-forward from the tensors under prefix p: 'dense' (SiLU-gated) or 'moe' (experts e0, e1, ... of that form stacked into one
-    matrix each way, an fp32 router, an optional shared expert with an optional one-row gate)."""
+    matrix each way, an fp32 router with an optional bias, an optional shared expert with an optional one-row gate).  chosen_softmax: the largest logits are chosen
+    and their soft-max weighs the experts' outputs (else a chosen expert's sigmoid score weighs its input)."""
     kind = mlp.get("kind")
     if kind == "dense":
         L.ff_kind, L.ff = FF_DENSE_SWIGLU, int(mlp["ff"])
@@ -222,6 +242,10 @@ def gated_feed_forward(L, st: SafeTensors, up, p: str, mlp: dict, width: int, wh
         L.ff_up = up.mat(np.concatenate([_gate_up(st, f"{p}e{e}.", L.ff, width, where) for e in range(L.experts)], axis=0))
         L.ff_down = up.mat(np.concatenate([st.bf16_bits(f"{p}e{e}.down") for e in range(L.experts)], axis=0))
         L.router = up.vec(_expect(st, p + "router", (L.experts, width)))
+        if p + "router.b" in st:
+            L.router_bias = up.vec(_expect(st, p + "router.b", (L.experts,)))
+        if chosen_softmax:
+            L.moe_softmax, L.moe_weight_output = 2, 1
         if mlp.get("shared"):
             L.shared_ff = int(mlp["shared"]["ff"])
             L.shared_up, L.shared_down = up.mat(_gate_up(st, p + "shared.", L.shared_ff, width, where)), up.mat(st.bf16_bits(p + "shared.down"))
@@ -294,9 +318,7 @@ def shared_key_latent_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str
     L.kv_rank, L.rot_dim = int(mc["kv_rank"]), int(mc["rot_dim"])
     rot = mc.get("rot") or {}
     L.rot_dims, L.rot_base = int(rot.get("dims") or 0), float(rot.get("base") or 10000.0)
-    sc = rot.get("scaling") or {}
-    if sc:
-        L.yarn_factor, L.yarn_fast, L.yarn_slow, L.yarn_original = float(sc["factor"]), float(sc["fast"]), float(sc["slow"]), int(sc["original"])
+    wavelength_scaling(L, rot)
     L.window, L.scale = int((mc.get("mask") or {}).get("size") or 0), float(mc["scale"])
     rows = [(m + "q", L.heads * (L.dim + L.rot_dim)), (m + "dkv", L.kv_rank + L.rot_dim)]
     if m + "g" in st:
@@ -470,6 +492,71 @@ def _pupidra_layers(cfg: dict, st: SafeTensors, up) -> tuple[list, dict]:
     return layers, top
 
 
+def matrix_memory_mixer(L, st: SafeTensors, up, m: str, mc: dict, where: str):
+    """Fill descriptor L with a matrix memory with exponential gates (MIX_MLSTM): q | k | v | g | i | f stacked with one bias vector (zeros where a projection has none)."""
+    L.kind = MIX_MLSTM
+    L.heads, L.dim = int(mc["heads"]), int(mc["dim"])
+    L.vdim, L.gate_cap = int(mc.get("vdim") or L.dim), float(mc.get("gate_cap") or 0.0)
+    rows = [(m + "q", L.heads * L.dim), (m + "k", L.heads * L.dim), (m + "v", L.heads * L.vdim), (m + "g", L.heads * L.vdim), (m + "i", L.heads), (m + "f", L.heads)]
+    for n, r in rows:
+        if st.shape(n)[0] != r:
+            raise ConfigError(f"tensor {n}: {st.shape(n)[0]} rows, the configuration gives {r} ({where})")
+    L.in_cat = up.mat(_stack(st, [n for n, _ in rows]))
+    if any(n + ".b" in st for n, _ in rows):
+        L.in_bias = up.vec(np.concatenate([_expect(st, n + ".b", (r,)) if n + ".b" in st else np.zeros(r, np.float32) for n, r in rows]))
+    L.onorm = up.vec(_expect(st, m + "norm", (L.heads * L.vdim,)))
+    L.out = up.mat(st.bf16_bits(m + "o"))
+
+
+def token_side_input(L, st: SafeTensors, up, p: str, dim: int, width: int, where: str):
+    """Fill descriptor L's per-layer token input from the tensors under prefix p"""
+    if st.shape(p + "gate") != (dim, width) or st.shape(p + "proj") != (width, dim):
+        raise ConfigError(f"{where}: token input shapes {st.shape(p + 'gate')} / {st.shape(p + 'proj')}, the configuration gives {(dim, width)}")
+    L.side_gate, L.side_proj = up.mat(st.bf16_bits(p + "gate")), up.mat(st.bf16_bits(p + "proj"))
+    L.side_norm = up.vec(_expect(st, p + "norm", (width,)))
+
+
+def _sogavik_layers(cfg: dict, st: SafeTensors, up) -> tuple[list, dict]:
+    width = int(cfg["width"])
+    side = cfg.get("token_side") or {}
+    layers, keep = [], []
+
+    def weight_and_bias(n):
+        return up.vec(_expect(st, n, (width,))), up.vec(_expect(st, n + ".b", (width,))) if n + ".b" in st else None
+
+    for i, lc in enumerate(cfg["layers"]):
+        p, mc, kind = f"l{i}.", lc["mixer"], lc["type"]
+        L = hip.SeqLayer()
+        L.form, L.mix_scale = LAYER_POSTNORM, 1.0
+        L.norm1b, L.norm1b_bias = weight_and_bias(p + "norm1")
+        if kind == "attention":
+            window_attention_mixer(L, st, up, p + "mix.", mc, f"layer {i}", ROT_HALVES, True)
+        elif kind == "parallel":
+            R = hip.SeqLayer()
+            window_attention_mixer(L, st, up, p + "mix.left.", mc["left"], f"layer {i} (left)", ROT_HALVES, True)
+            matrix_memory_mixer(R, st, up, p + "mix.right.", mc["right"], f"layer {i} (right)")
+            L.mix_onorm, R.mix_onorm = (up.vec(_expect(st, p + "mix." + s + ".out", (width,))) for s in ("left", "right"))
+            L.mix_scale = R.mix_scale = 0.5
+            keep.append(R)
+            L.beside = C.pointer(R)
+        else:
+            raise ConfigError(f"layer {i}: mixer type {kind!r} is not known")
+        if lc.get("mlp"):
+            L.norm2b, L.norm2b_bias = weight_and_bias(p + "norm2")
+            gated_feed_forward(L, st, up, p + "mlp.", lc["mlp"], width, f"layer {i}", chosen_softmax=True)
+        if side:
+            token_side_input(L, st, up, p + "side.", int(side["dim"]), width, f"layer {i}")
+        layers.append(L)
+    norm, bias = weight_and_bias("final.norm")
+    top = dict(width=width, vocab=int(cfg["vocab"]), canon_taps=1, norm_eps=float(cfg["norm"]["eps"]), norm_offset=0.0, norm_center=1, logit_scale=1.0,
+               embed=up.mat(st.bf16_bits("embed")), head=up.mat(st.bf16_bits("head")), final_norm=norm, final_norm_bias=bias, _keep=keep)
+    if side:
+        if st.shape("side.embed") != (int(cfg["vocab"]), len(layers) * int(side["dim"])):
+            raise ConfigError(f"tensor side.embed: shape {st.shape('side.embed')}, the configuration gives {(int(cfg['vocab']), len(layers) * int(side['dim']))}")
+        top.update(side_embed=up.mat(st.bf16_bits("side.embed")), side_dim=int(side["dim"]))
+    return layers, top
+
+
 def _vobisun_layers(cfg: dict, st: SafeTensors, up) -> tuple[list, dict]:
     width = int(cfg["width"])
     taps = int((cfg.get("canon") or {}).get("taps") or 1)
@@ -509,7 +596,8 @@ def _vobisun_layers(cfg: dict, st: SafeTensors, up) -> tuple[list, dict]:
     return layers, top
 
 
-ARCHITECTURES = {"Ranutar": _ranutar_layers, "Vobisun": _vobisun_layers, "Zusolix": _zusolix_layers, "Pokatar": _pokatar_layers, "Pupidra": _pupidra_layers}
+ARCHITECTURES = {"Ranutar": _ranutar_layers, "Vobisun": _vobisun_layers, "Zusolix": _zusolix_layers, "Pokatar": _pokatar_layers, "Pupidra": _pupidra_layers,
+                 "Sogavik": _sogavik_layers}
 
 
 def read_config(model_dir: str) -> dict:

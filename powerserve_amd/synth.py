@@ -522,11 +522,94 @@ def _pupidra_tensors(cfg: dict, seed: int) -> dict:
     return t
 
 
+def sogavik_attention(heads: int, kv_heads: int, dim: int, vdim: int, scale: float, size: int, dims: int, base: float = 10000.0, scaling: tuple | None = None) -> dict:
+    """mixer entry of a Sogavik attention layer (or of a parallel layer's left side); scaling: (factor, original, fast, slow) or None"""
+    rot = {"base": float(base), "dims": int(dims)}
+    if scaling:
+        rot["scaling"] = {"factor": float(scaling[0]), "original": int(scaling[1]), "fast": float(scaling[2]), "slow": float(scaling[3])}
+    return {"heads": int(heads), "kv_heads": int(kv_heads), "dim": int(dim), "vdim": int(vdim), "scale": float(scale), "mask": {"size": int(size)}, "rot": rot}
+
+
+def sogavik_memory(heads: int, dim: int, vdim: int, gate_cap: float) -> dict:
+    """the right side of a Sogavik parallel layer"""
+    return {"heads": int(heads), "dim": int(dim), "vdim": int(vdim), "gate_cap": float(gate_cap)}
+
+
+def sogavik_layer(mixer: dict, right: dict | None = None, moe: tuple | None = None) -> dict:
+    """One entry of a Sogavik configuration's 'layers': an attention layer, or (right given) a parallel one; moe = (experts, top, expert ff) or None."""
+    mlp = {"kind": "moe", "router": {"experts": int(moe[0]), "top": int(moe[1])}, "expert": {"ff": int(moe[2])}} if moe else None
+    return {"type": "parallel", "mixer": {"left": dict(mixer), "right": dict(right)}, "mlp": mlp} if right else {"type": "attention", "mixer": dict(mixer), "mlp": mlp}
+
+
+def sogavik_config(width: int, vocab: int, layers: list, side: int | None, eps: float = 1e-6) -> dict:
+    cfg = {"architecture": "Sogavik", "layers": layers, "norm": {"eps": float(eps)}, "vocab": int(vocab), "width": int(width)}
+    if side:
+        cfg["token_side"] = {"dim": int(side)}
+    return cfg
+
+
+def _sogavik_tensors(cfg: dict, seed: int) -> dict:
+    rng = np.random.default_rng(seed)
+    W = cfg["width"]
+
+    def lin(n, k, gain=1.0):
+        return rng.standard_normal((n, k), dtype=np.float32) * np.float32(gain / np.sqrt(k))
+
+    def vec(n, std=0.1, mean=0.0):
+        return (rng.standard_normal(n, dtype=np.float32) * np.float32(std) + np.float32(mean)).astype(np.float32)
+
+    t = {"embed": rng.standard_normal((cfg["vocab"], W), dtype=np.float32)}
+
+    def norm(n):
+        t[n], t[n + ".b"] = vec(W, 0.2, 1.0), vec(W, 0.2)
+
+    def attention(m, mc, gate):
+        H, G, d, dv = mc["heads"], mc["kv_heads"], mc["dim"], mc["vdim"]
+        for n, r in (("q", H * d), ("k", G * d), ("v", G * dv)):
+            t[m + n], t[m + n + ".b"] = lin(r, W), vec(r, 0.3)
+        t[m + "q.norm"], t[m + "k.norm"], t[m + "o"] = vec(H * d, 0.3, 1.0), vec(G * d, 0.3, 1.0), lin(W, H * dv)
+        if gate:
+            t[m + "g"] = lin(H, W, 1.5)
+
+    side = (cfg.get("token_side") or {}).get("dim")
+    if side:
+        t["side.embed"] = rng.standard_normal((cfg["vocab"], len(cfg["layers"]) * side), dtype=np.float32)
+    for i, lc in enumerate(cfg["layers"]):
+        p, m, mc = f"l{i}.", f"l{i}.mix.", lc["mixer"]
+        norm(p + "norm1")
+        if lc["type"] == "attention":
+            attention(m, mc, True)
+        elif lc["type"] == "parallel":
+            attention(m + "left.", mc["left"], False)
+            r, mr = mc["right"], m + "right."
+            H, d, dv = r["heads"], r["dim"], r["vdim"]
+            for n, rows in (("q", H * d), ("k", H * d), ("v", H * dv), ("g", H * dv)):
+                t[mr + n] = lin(rows, W)
+            # gates: a few nats of spread, memories from a few tokens to hundreds
+            t[mr + "i"], t[mr + "i.b"], t[mr + "f"], t[mr + "f.b"] = lin(H, W), vec(H, 1.0, -1.0), lin(H, W), vec(H, 1.0, 3.5)
+            t[mr + "norm"], t[mr + "o"] = vec(H * dv, 0.2, 1.0), lin(W, H * dv)
+            t[m + "left.out"], t[m + "right.out"] = vec(W, 0.2, 1.0), vec(W, 0.2, 1.0)
+        else:
+            raise ValueError(lc["type"])
+        mlp = lc.get("mlp")
+        if mlp:
+            norm(p + "norm2")
+            q, ff = p + "mlp.", mlp["expert"]["ff"]
+            for e in range(mlp["router"]["experts"]):
+                t[f"{q}e{e}.gate"], t[f"{q}e{e}.up"], t[f"{q}e{e}.down"] = lin(ff, W), lin(ff, W), lin(W, ff)
+            t[q + "router"], t[q + "router.b"] = lin(mlp["router"]["experts"], W), vec(mlp["router"]["experts"], 0.5)
+        if side:
+            t[p + "side.gate"], t[p + "side.proj"], t[p + "side.norm"] = lin(side, W), lin(W, side), vec(W, 0.2, 0.6)
+    norm("final.norm")
+    t["head"] = lin(cfg["vocab"], W)
+    return t
+
+
 def seq_tensors(cfg: dict, seed: int = 0, decay_rank: int = 8) -> dict:
     """Random-init tensors of a layer-list configuration, name -> float32 array already rounded to bfloat16 (what the file will hold)."""
     from .safetensors_io import f32_to_bf16_bits
     makers = {"Vobisun": lambda: _parallel_tensors(cfg, seed, decay_rank), "Zusolix": lambda: _zusolix_tensors(cfg, seed), "Pokatar": lambda: _pokatar_tensors(cfg, seed),
-              "Pupidra": lambda: _pupidra_tensors(cfg, seed)}
+              "Pupidra": lambda: _pupidra_tensors(cfg, seed), "Sogavik": lambda: _sogavik_tensors(cfg, seed)}
     if cfg.get("architecture") in makers:
         t = makers[cfg["architecture"]]()
         return {k: (f32_to_bf16_bits(v).astype(np.uint32) << 16).view(np.float32).reshape(v.shape) for k, v in t.items()}

@@ -739,3 +739,150 @@ def run_pupidra(cfg, W, tokens, per_layer=None, use_bigram=True, use_previous=Tr
     logits = plain_norm(x, W["final.norm"], eps) @ W["head"].T
     cap = cfg.get("logit_softcap")
     return cap * np.tanh(logits / cap) if cap and use_cap else logits
+
+
+# ------------------------------------------------------------------------------------------------ Sogavik
+# Post-norm layers with layer norms that have a weight and a bias,  x += ln1(mixer(x));  x += ln2(ff(x)), then a per-layer input taken from the token itself:
+# x += rms(P (gelu(G x) * e)) w  with e the layer's stretch of a second embedding row.  Mixers: grouped-query attention over a sliding window with biases on q, k
+# and v, RMS norms over the whole q / k projections, rotate-half rotary (frequencies scaled by wavelength) on the first numbers of a head and a gate per head; or
+# two mixers side by side -- such an attention, ungated, and a matrix memory with exponential gates -- whose outputs are RMS-normed one by one and averaged.  The
+# feed-forward is a mixture of SiLU-gated experts, the chosen logits' soft-max on their outputs.
+
+
+def biased_layer_norm(a, w, b, eps, use_mean=True):
+    return (centred_norm(a, w, eps) if use_mean else plain_norm(a, w, eps)) + b
+
+
+def gelu_tanh(z):
+    return 0.5 * z * (1.0 + np.tanh(np.sqrt(2.0 / np.pi) * (z + 0.044715 * z ** 3)))
+
+
+def token_side_input(W, pre, x, tokens, layer, dim, eps, use_gate=True, shift=0):
+    """What layer number `layer` adds for the tokens themselves.  shift: a WRONG model that reads another layer's stretch of the table."""
+    at = (layer + shift) * dim
+    e = W["side.embed"][np.asarray(tokens), at:at + dim]
+    y = ((gelu_tanh(x @ W[pre + "gate"].T) if use_gate else 1.0) * e) @ W[pre + "proj"].T
+    return unit_rms(y, eps) * W[pre + "norm"]
+
+
+def normed_window_attention(W, pre, h, mc, eps, size=None, use_bias=True, use_norm=True, per_head=False, use_rotation=True, use_scaling=True, use_gate=True):
+    """size: a WRONG window; per_head: a WRONG norm taken over each head instead of the whole projection."""
+    T = h.shape[0]
+    H, G, d, dv = mc["heads"], mc["kv_heads"], mc["dim"], mc["vdim"]
+    size = mc["mask"]["size"] if size is None else size
+
+    def proj(n):
+        return h @ W[pre + n].T + (W[pre + n + ".b"] if use_bias else 0.0)
+
+    def normed(a, w, heads):
+        if not use_norm:
+            return a.reshape(T, heads, d)
+        return ((unit_rms(a.reshape(T, heads, d), eps).reshape(T, -1) if per_head else unit_rms(a, eps)) * w).reshape(T, heads, d)
+
+    q, k, v = normed(proj("q"), W[pre + "q.norm"], H), normed(proj("k"), W[pre + "k.norm"], G), proj("v").reshape(T, G, dv)
+    if use_rotation:
+        rot = dict(mc["rot"])
+        if not use_scaling:
+            rot.pop("scaling", None)
+        freqs, mag = yarn_frequencies(rot)
+        q = np.stack([rotate_halves(q[t], t, freqs, mag) for t in range(T)])
+        k = np.stack([rotate_halves(k[t], t, freqs, mag) for t in range(T)])
+    visible = kept_window_mask(T, size, 0)
+    gate = sigmoid(h @ W[pre + "g"].T) if use_gate and pre + "g" in W else np.ones((T, H))
+    out = np.zeros((T, H, dv))
+    for hd in range(H):
+        g = hd // (H // G)
+        s = np.where(visible, q[:, hd] @ k[:, g].T * mc["scale"], -np.inf)
+        e = np.exp(s - s.max(axis=1, keepdims=True))
+        out[:, hd] = e / e.sum(axis=1, keepdims=True) @ v[:, g] * gate[:, hd:hd + 1]
+    return out.reshape(T, H * dv) @ W[pre + "o"].T
+
+
+def matrix_memory_scan(q, k, v, i, f, m0=0.0, carry=True, lose_at=None, use_floor=True):
+    """q (scaled), k [T, H, d], v [T, H, dv], i / f [T, H] the logarithms of the input and forget gates; S, n zero and the running maximum m0 in front of the
+    first token.  lose_at: a WRONG model whose state is lost in front of that token (carry False: of every token); use_floor False: ... without the floor of the
+    denominator."""
+    T, H, d = q.shape
+    out = np.zeros(v.shape)
+    for hd in range(H):
+        S, n, m = np.zeros((d, v.shape[2])), np.zeros(d), m0
+        for t in range(T):
+            if not carry or t == lose_at:
+                S, n, m = np.zeros_like(S), np.zeros(d), m0
+            new = max(f[t, hd] + m, i[t, hd])
+            a, b = np.exp(f[t, hd] + m - new), np.exp(i[t, hd] - new)
+            S = a * S + b * np.outer(k[t, hd], v[t, hd])
+            n = a * n + b * k[t, hd]
+            m = new
+            low = abs(n @ q[t, hd])
+            out[t, hd] = S.T @ q[t, hd] / ((max(low, np.exp(-m)) if use_floor else low) + 1e-6)
+    return out
+
+
+def capped(z, cap):
+    return cap * np.tanh(z / cap)
+
+
+def log_sigmoid(z):
+    return -softplus(-z)
+
+
+def matrix_memory_mixer(W, pre, h, mc, eps, use_cap=True, use_norm=True, use_gate=True, **scan_kw):
+    T = h.shape[0]
+    H, d, dv = mc["heads"], mc["dim"], mc["vdim"]
+    q, k, v = (h @ W[pre + "q"].T).reshape(T, H, d) * d ** -0.5, (h @ W[pre + "k"].T).reshape(T, H, d), (h @ W[pre + "v"].T).reshape(T, H, dv)
+    cap = (lambda z: capped(z, mc["gate_cap"])) if use_cap else (lambda z: z)
+    i, f = cap(h @ W[pre + "i"].T + W[pre + "i.b"]), log_sigmoid(cap(h @ W[pre + "f"].T + W[pre + "f.b"]))
+    o = matrix_memory_scan(q, k, v, i, f, **scan_kw)
+    o = (unit_rms(o, eps) if use_norm else o).reshape(T, H * dv) * W[pre + "norm"]
+    return (o * sigmoid(h @ W[pre + "g"].T) if use_gate else o) @ W[pre + "o"].T
+
+
+def averaged_pair_mixer(W, pre, h, mc, eps, left_kw=None, right_kw=None, use_out_norms=True, use_left=True, use_right=True):
+    a = normed_window_attention(W, pre + "left.", h, mc["left"], eps, **(left_kw or {}))
+    b = matrix_memory_mixer(W, pre + "right.", h, mc["right"], eps, **(right_kw or {}))
+    if use_out_norms:
+        a, b = plain_norm(a, W[pre + "left.out"], eps), plain_norm(b, W[pre + "right.out"], eps)
+    return 0.5 * ((a if use_left else 0.0) + (b if use_right else 0.0))
+
+
+def chosen_softmax_experts(W, pre, h, mlp, use_bias=True, over_all=False):
+    """over_all: a WRONG model whose weights are the chosen shares of the soft-max over every expert."""
+    r = mlp["router"]
+    out = np.zeros_like(h)
+    for t in range(h.shape[0]):
+        z = W[pre + "router"] @ h[t] + (W[pre + "router.b"] if use_bias else 0.0)
+        chosen = np.argsort(-z, kind="stable")[:r["top"]]
+        w = np.exp(z - z.max())
+        w = w / (w.sum() if over_all else w[chosen].sum())
+        for e in chosen:
+            p = f"{pre}e{e}."
+            out[t] += w[e] * (W[p + "down"] @ (silu(W[p + "gate"] @ h[t]) * (W[p + "up"] @ h[t])))
+    return out
+
+
+def run_sogavik(cfg, W, tokens, per_layer=None, use_mean=True, use_norm_bias=True, use_side=True, side_kw=None, attn_kw=None, pair_kw=None, moe_kw=None):
+    """-> logits [T, vocab]; per_layer (a list) receives the residual stream after every layer."""
+    W = {k: np.asarray(v, dtype=np.float64) for k, v in W.items()}
+    eps = cfg["norm"]["eps"]
+    x = W["embed"][np.asarray(tokens)]
+
+    def norm(a, n):
+        return biased_layer_norm(a, W[n], W[n + ".b"] if use_norm_bias else 0.0, eps, use_mean)
+
+    for i, lc in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        if lc["type"] == "attention":
+            y = normed_window_attention(W, p + "mix.", x, lc["mixer"], eps, **(attn_kw or {}))
+        elif lc["type"] == "parallel":
+            y = averaged_pair_mixer(W, p + "mix.", x, lc["mixer"], eps, **(pair_kw or {}))
+        else:
+            raise ValueError(lc["type"])
+        x = x + norm(y, p + "norm1")
+        if lc.get("mlp"):
+            x = x + norm(chosen_softmax_experts(W, p + "mlp.", x, lc["mlp"], **(moe_kw or {})), p + "norm2")
+        if use_side and cfg.get("token_side"):
+            x = x + token_side_input(W, p + "side.", x, tokens, i, cfg["token_side"]["dim"], eps, **(side_kw or {}))
+        if per_layer is not None:
+            per_layer.append(x.copy())
+    return norm(x, "final.norm") @ W["head"].T
