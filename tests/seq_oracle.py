@@ -757,9 +757,9 @@ def gelu_tanh(z):
     return 0.5 * z * (1.0 + np.tanh(np.sqrt(2.0 / np.pi) * (z + 0.044715 * z ** 3)))
 
 
-def token_side_input(W, pre, x, tokens, layer, dim, eps, use_gate=True, shift=0):
-    """What layer number `layer` adds for the tokens themselves.  shift: a WRONG model that reads another layer's stretch of the table."""
-    at = (layer + shift) * dim
+def token_side_input(W, pre, x, tokens, layer, dim, eps, use_gate=True):
+    """What layer number `layer` adds for the tokens themselves."""
+    at = layer * dim
     e = W["side.embed"][np.asarray(tokens), at:at + dim]
     y = ((gelu_tanh(x @ W[pre + "gate"].T) if use_gate else 1.0) * e) @ W[pre + "proj"].T
     return unit_rms(y, eps) * W[pre + "norm"]
@@ -846,18 +846,20 @@ def averaged_pair_mixer(W, pre, h, mc, eps, left_kw=None, right_kw=None, use_out
     return 0.5 * ((a if use_left else 0.0) + (b if use_right else 0.0))
 
 
-def chosen_softmax_experts(W, pre, h, mlp, use_bias=True, over_all=False):
-    """over_all: a WRONG model whose weights are the chosen shares of the soft-max over every expert."""
+def chosen_softmax_experts(W, pre, h, mlp, use_bias=True, equal=False, on_input=False):
+    """equal, on_input: WRONG models whose chosen experts count alike, or whose weights multiply what an expert reads.  (Shares of the soft-max over ALL experts would differ by
+    one factor per token only, which the norm behind the sublayer takes out again.)"""
     r = mlp["router"]
     out = np.zeros_like(h)
     for t in range(h.shape[0]):
         z = W[pre + "router"] @ h[t] + (W[pre + "router.b"] if use_bias else 0.0)
         chosen = np.argsort(-z, kind="stable")[:r["top"]]
         w = np.exp(z - z.max())
-        w = w / (w.sum() if over_all else w[chosen].sum())
+        w = np.full(len(z), 1.0 / len(chosen)) if equal else w / w[chosen].sum()
         for e in chosen:
             p = f"{pre}e{e}."
-            out[t] += w[e] * (W[p + "down"] @ (silu(W[p + "gate"] @ h[t]) * (W[p + "up"] @ h[t])))
+            a = h[t] * (w[e] if on_input else 1.0)
+            out[t] += (1.0 if on_input else w[e]) * (W[p + "down"] @ (silu(W[p + "gate"] @ a) * (W[p + "up"] @ a)))
     return out
 
 

@@ -457,3 +457,105 @@ def test_the_small_library_exports_what_its_models_need():
         pytest.skip("lib/libps_hip_seq.so not built")
     lib = C.CDLL(hip.SEQ_LIB_PATH)
     assert not [n for n in hip.SEQ_EXPORTS if not hasattr(lib, n)]
+
+
+SCFG = synth.sogavik_config(24, 30, [
+    synth.sogavik_layer(synth.sogavik_attention(4, 2, 6, 10, 0.25, 9, 4, 100.0, (4.0, 40, 8.0, 0.5)), moe=(3, 2, 8)),
+    synth.sogavik_layer(synth.sogavik_attention(3, 3, 6, 5, 0.5, 7, 2, 77.0), synth.sogavik_memory(5, 4, 3, 6.0), (4, 1, 6)),
+    synth.sogavik_layer(synth.sogavik_attention(2, 1, 6, 10, 0.25, 5, 6))], side=5, eps=1e-5)
+
+
+def test_sogavik_configuration_maps_onto_layer_descriptors(tmp_path):
+    t = synth.write_seq_model_dir(str(tmp_path), SCFG, 1)
+    cfg = seqmodel.read_config(str(tmp_path))
+    up = FakeUp()
+    st = safetensors_io.SafeTensors(str(tmp_path / "model.safetensors"))
+    layers, top = seqmodel.ARCHITECTURES[cfg["architecture"]](cfg, st, up)
+    bits = safetensors_io.f32_to_bf16_bits
+    assert (top["width"], top["vocab"], top["norm_offset"], top["norm_center"], top["side_dim"]) == (24, 30, 0.0, 1, 5) and top["head"] != top["embed"]
+    assert up.mats[top["side_embed"] - 1001].shape == (30, 15) and np.array_equal(up.vecs[top["final_norm_bias"] - 1], t["final.norm.b"])
+    a, b, c = layers
+    for i, x in enumerate(layers):
+        assert x.form == seqmodel.LAYER_POSTNORM and x.norm1 is None and x.norm2 is None and x.canon1 is None
+        assert np.array_equal(up.vecs[x.norm1b - 1], t[f"l{i}.norm1"]) and np.array_equal(up.vecs[x.norm1b_bias - 1], t[f"l{i}.norm1.b"])
+        assert up.mats[x.side_gate - 1001].shape == (5, 24) and up.mats[x.side_proj - 1001].shape == (24, 5) and np.array_equal(up.vecs[x.side_norm - 1], t[f"l{i}.side.norm"])
+    assert np.array_equal(up.vecs[a.norm2b_bias - 1], t["l0.norm2.b"]) and c.norm2b is None and c.ff_kind == seqmodel.FF_NONE
+    # attention: q | k | v | gate stacked, biases alike (none for the gate), norms over the whole projections, frequencies scaled by wavelength
+    assert (a.kind, a.heads, a.kv_heads, a.dim, a.vdim, a.window, a.rot_dims, a.rot_pairing, a.gated, a.head_norm, a.yarn_factor, a.yarn_original, a.yarn_fast, a.yarn_slow) == (
+        seqmodel.MIX_WINATTN, 4, 2, 6, 10, 9, 4, seqmodel.ROT_HALVES, 1, 0, 4.0, 40, 8.0, 0.5)
+    assert np.array_equal(up.mats[a.in_cat - 1001], np.concatenate([bits(t["l0.mix." + n]) for n in "qkvg"]))
+    assert np.array_equal(up.vecs[a.in_bias - 1], np.concatenate([t["l0.mix." + n + ".b"] for n in "qkv"] + [np.zeros(4, np.float32)]))
+    assert up.vecs[a.qnorm - 1].shape == (24,) and up.vecs[a.knorm - 1].shape == (12,) and not a.beside and a.mix_scale == 1.0 and a.mix_onorm is None
+    # the pair: half of each side's output behind a norm of its own
+    r = b.beside.contents
+    assert (b.kind, b.gated, b.yarn_factor, b.mix_scale, r.mix_scale) == (seqmodel.MIX_WINATTN, 0, 0.0, 0.5, 0.5)
+    assert np.array_equal(up.vecs[b.mix_onorm - 1], t["l1.mix.left.out"]) and np.array_equal(up.vecs[r.mix_onorm - 1], t["l1.mix.right.out"])
+    assert (r.kind, r.heads, r.dim, r.vdim, r.gate_cap) == (seqmodel.MIX_MLSTM, 5, 4, 3, 6.0)
+    assert np.array_equal(up.mats[r.in_cat - 1001], np.concatenate([bits(t["l1.mix.right." + n]) for n in "qkvgif"]))
+    assert np.array_equal(up.vecs[r.in_bias - 1], np.concatenate([np.zeros(70, np.float32), t["l1.mix.right.i.b"], t["l1.mix.right.f.b"]])) and up.vecs[r.onorm - 1].shape == (15,)
+    # the experts
+    assert (a.ff_kind, a.ff, a.experts, a.top, a.moe_softmax, a.moe_weight_output, a.moe_norm_top, b.top) == (seqmodel.FF_MOE_SWIGLU, 8, 3, 2, 2, 1, 0, 1)
+    assert np.array_equal(up.vecs[a.router_bias - 1], t["l0.mlp.router.b"]) and up.mats[a.ff_up - 1001].shape == (48, 24)
+    # what the file and the configuration do not have does not exist
+    less = {n: st.f32(n) for n in st.names() if not n.endswith(".b") and "side." not in n and n != "l0.mix.g"}
+    cfg2 = json.loads(json.dumps(SCFG))
+    del cfg2["token_side"], cfg2["layers"][0]["mixer"]["rot"]["scaling"]
+    synth.write_seq_model_dir(str(tmp_path / "less"), cfg2, 1, tensors=less)
+    layers, top = seqmodel.ARCHITECTURES["Sogavik"](cfg2, safetensors_io.SafeTensors(str(tmp_path / "less" / "model.safetensors")), FakeUp())
+    a, b, c = layers
+    assert "side_embed" not in top and top["final_norm_bias"] is None and (a.side_gate, a.norm1b_bias, a.in_bias, a.router_bias, a.gated, a.yarn_factor, b.beside.contents.in_bias) == (
+        None, None, None, None, 0, 0.0, None)
+    for i, path, val in ((0, ("type",), "conveyor"), (0, ("mlp",), {"kind": "sparse", "ff": 8}), (0, ("mixer", "kv_heads"), 3), (0, ("mixer", "dim"), 7), (1, ("mixer", "right", "heads"), 4),
+                         (1, ("mixer", "right", "vdim"), 4), (0, ("mlp", "router", "top"), 4)):
+        bad = json.loads(json.dumps(SCFG))
+        at = bad["layers"][i]
+        for k in path[:-1]:
+            at = at[k]
+        at[path[-1]] = val
+        with pytest.raises(seqmodel.ConfigError):
+            seqmodel.ARCHITECTURES["Sogavik"](bad, st, FakeUp())
+    for val in (4, 6):
+        with pytest.raises(seqmodel.ConfigError):
+            seqmodel.ARCHITECTURES["Sogavik"](dict(SCFG, token_side={"dim": val}), st, FakeUp())
+
+
+def test_plain_sogavik_statement_reach_and_pieces():
+    """causal; the layer norm takes the mean off in front of its bias; the memory against its closed form, with a denominator that has a floor; the running maximum changes nothing but the
+    range; the chosen soft-max; the side input reads the layer's own stretch"""
+    t = synth.seq_tensors(SCFG, 2)
+    rng = np.random.default_rng(0)
+    a = rng.integers(0, 30, 20)
+    b = a.copy()
+    b[6] = (b[6] + 1) % 30
+    la, lb = seq_oracle.run_sogavik(SCFG, t, a), seq_oracle.run_sogavik(SCFG, t, b)
+    assert np.array_equal(la[:6], lb[:6]) and min(np.abs(la[i] - lb[i]).max() for i in range(6, 20)) > 1e-6
+    x = rng.standard_normal((4, 12))
+    n = seq_oracle.biased_layer_norm(x + 3.0, np.ones(12), 0.25, 1e-9)
+    assert np.allclose(n.mean(-1), 0.25) and np.allclose(np.var(n, axis=-1), 1.0)
+    z = np.linspace(-4, 4, 9)
+    assert np.allclose(seq_oracle.gelu_tanh(z) - seq_oracle.gelu_tanh(-z), z) and seq_oracle.gelu_tanh(np.float64(1.0)) == pytest.approx(0.841192, abs=1e-6)
+    assert np.allclose(seq_oracle.log_sigmoid(z), np.log(1 / (1 + np.exp(-z)))) and abs(seq_oracle.capped(1e9, 5.0) - 5.0) < 1e-12
+    # o_t = sum_s D_ts (q_t . k_s) v_s / (max(|sum_s D_ts (q_t . k_s)|, 1) + tiny),  D_ts = exp(f_(s+1) + .. + f_t + i_s): the maximum cancels but for the 1e-6
+    T, H, d, dv = 9, 2, 3, 4
+    q, k, v = rng.standard_normal((T, H, d)), rng.standard_normal((T, H, d)), rng.standard_normal((T, H, dv))
+    i, f = rng.standard_normal((T, H)), seq_oracle.log_sigmoid(rng.standard_normal((T, H)))
+    o = seq_oracle.matrix_memory_scan(q, k, v, i, f)
+    for h in range(H):
+        c = np.cumsum(f[:, h])
+        for s in range(T):
+            w = np.exp(c[s] - c[:s + 1] + i[:s + 1, h]) * (k[:s + 1, h] @ q[s, h])
+            assert np.allclose(o[s, h], w @ v[:s + 1, h] / max(abs(w.sum()), 1.0), rtol=1e-4, atol=1e-6)
+    assert np.allclose(o, seq_oracle.matrix_memory_scan(q, k, v, i, f, m0=-50.0), rtol=1e-4, atol=1e-6)
+    W = {n: np.asarray(u, np.float64) for n, u in t.items()}
+    h = rng.standard_normal((5, 24))
+    moe = SCFG["layers"][0]["mlp"]
+    got = seq_oracle.chosen_softmax_experts(W, "l0.mlp.", h, moe)
+    for r in range(5):
+        zr = W["l0.mlp.router"] @ h[r] + W["l0.mlp.router.b"]
+        e0, e1 = np.argsort(-zr)[:2]
+        w0 = 1.0 / (1.0 + np.exp(zr[e1] - zr[e0]))
+        y = [seq_oracle.gated_feed_forward(W, f"l0.mlp.e{e}.", h[r]) for e in (e0, e1)]
+        assert np.allclose(got[r], w0 * y[0] + (1 - w0) * y[1])
+    u = seq_oracle.token_side_input(W, "l1.side.", h, a[:5], 1, 5, 1e-5)
+    other = dict(W, **{"side.embed": np.where(np.arange(15) // 5 == 1, W["side.embed"], 0.0)})
+    assert np.allclose(u, seq_oracle.token_side_input(other, "l1.side.", h, a[:5], 1, 5, 1e-5)) and np.allclose(np.mean((u / W["l1.side.norm"]) ** 2, axis=-1), 1.0, atol=1e-3)
