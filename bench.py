@@ -58,7 +58,8 @@ def parse():
                     "the sizes z2048x6 / z4096x3 (Zusolix: depth-averaged parallel layers, soft-capped causal attention or a gated recurrence, mixture-of-experts feed-forwards) "
                     "beside the v sizes, the sizes p2048x6 / p4096x3 (Pokatar: pre-norm layers, sink attention or shared-key latent attention, relu-gated dense and "
                     "squared-relu expert feed-forwards) beside the z sizes, the sizes u2048x6 / u4096x3 (Pupidra: post-norm layers, state-space recurrence, windowed attention with "
-                    "first tokens and shared keys, latent attention, squared-relu experts) beside the p sizes")
+                    "first tokens and shared keys, latent attention, squared-relu experts) beside the p sizes, the sizes s2048x6 / s4096x3 (Sogavik: post-norm layers with a token input "
+                    "each, windowed attention alone or averaged with a matrix memory, SiLU-gated experts) beside the u sizes")
     ap.add_argument("--layer-list-portion", type=int, default=512, help="--layer-list: tokens per launch sequence of the prefill")
     ap.add_argument("--prefill-warmup-tokens", type=int, default=128, help="untimed tokens forwarded before the timed prefill (first use of the prefill kernels in the process; 0: none)")
     ap.add_argument("--wide-chunk", type=int, default=512, help="side leg: prefill in chunks of this many tokens (0: skip)")

@@ -43,11 +43,25 @@ SIZES = {
                     top=2, order="mmalsl", layers=6, beside="p2048x6"),
     "u4096x3": dict(design="Pupidra", width=4096, ff=14336, heads=32, kv_heads=8, dim=128, window=1024, keep_first=64, kv_rank=512, rot_dim=64, state=128, groups=8, experts=8,
                     top=2, order="mal", layers=3, beside="p4096x3"),
+    # Sogavik (post-norm layers with biased layer norms and a token input of 256 numbers per layer; a = windowed attention with wavelength-scaled rotary and a gate per head, p = such an
+    # attention beside a matrix memory with keys of 128 and values of 256 -- the Pupidra recurrence's bytes of state; every feed-forward 8 SiLU-gated experts, top 2: three matrices per
+    # expert and no shared one, so an inner size of ff / 2 makes a token use the Pupidra layers' feed-forward weights) beside the Pupidra model of equal width, heads, window and layers
+    "s2048x6": dict(design="Sogavik", width=2048, ff=8192, heads=16, kv_heads=4, dim=128, window=1024, rot_dims=64, mem_heads=16, mem_dim=128, mem_vdim=256, side=256, experts=8, top=2,
+                    order="apapap", layers=6, beside="u2048x6"),
+    "s4096x3": dict(design="Sogavik", width=4096, ff=14336, heads=32, kv_heads=8, dim=128, window=1024, rot_dims=64, mem_heads=32, mem_dim=128, mem_vdim=256, side=256, experts=8, top=2,
+                    order="apa", layers=3, beside="u4096x3"),
 }
 
 
 def config(z: dict, vocab: int = 4096) -> dict:
     H, d = z["heads"], z["dim"]
+    if z.get("design") == "Sogavik":
+        scale = float(d ** -0.5)
+        att = synth.sogavik_attention(H, z["kv_heads"], d, d, scale, z["window"], z["rot_dims"], 5e5, (4.0, 4096, 24.0, 1.5))
+        left = synth.sogavik_attention(H, z["kv_heads"], d, d, scale, z["window"], z["rot_dims"], 1e4)
+        right = synth.sogavik_memory(z["mem_heads"], z["mem_dim"], z["mem_vdim"], 15.0)
+        moe = (z["experts"], z["top"], z["ff"] // 2)
+        return synth.sogavik_config(z["width"], vocab, [synth.sogavik_layer(att, moe=moe) if k == "a" else synth.sogavik_layer(left, right, moe) for k in z["order"]], side=z["side"])
     if z.get("design") == "Pupidra":
         kinds = {"m": ("mamba2", synth.pupidra_mamba2(2 * z["width"] // 64, 64, z["state"], z["groups"], 4, z["groups"])),
                  "l": ("latent_attention", synth.pupidra_latent(H, d, z["rot_dim"], d, z["kv_rank"], float((d + z["rot_dim"]) ** -0.5), 5e5))}

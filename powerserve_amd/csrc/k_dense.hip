@@ -2,7 +2,8 @@
 // fp32 throughout on v_mfma_f32_16x16x4_f32 (one rounding per product, fp32 adds: a true fp32 product, no reduced-precision mode).
 //   dense_mm_kernel<WT>   tiled mat-mul, 64 tokens x 64 outputs per work-group of four waves, any T / N / K (edges zero-filled)
 //   dense_mm_fast_kernel  bf16, K % 64 == 0, more than 8 tokens: 128 x 128 tiles over an operand packed to bf16 by dense_pack_kernel
-//   dense_mv_kernel<WT,C> a few tokens (C <= 8 columns): the activation rows live in LDS, a wave streams four weight rows at a time
+//   dense_mm_narrow_kernel bf16, K % 128 == 0, more than 8 tokens, products too small to fill the chip with 128 x 128 tiles: 32 x 32 tiles, the four waves share K
+//   dense_mv_kernel<WT,C,RW> a few tokens (C <= 8 columns): the activation rows live in LDS, a wave streams RW weight rows at a time
 // All take the same operand description (ps_seq.h psk_dense_args): ring rows, the token-shift mix and the epilogue
 // (bias, activation, scale, a factor from a second table) are part of the launch, so no mixer needs a kernel of its own around its projections.
 #include "ps_seq.h"
@@ -222,24 +223,28 @@ __global__ __launch_bounds__(256) void dense_mm_kernel(dn_args g) {
 
 // ---------------------------------------------------------------------------------------------------- a few tokens: mat-vec
 // Dynamic LDS: C rows of K activations, as bf16-rounded fp32 values (bf16 mode: the same operand rounding as the tiled kernel) or fp32.
-template <typename WT, int C>
+template <typename WT, int C, int RW> // RW rows per wave at a time: four, or one where four would leave most of the chip without a wave (no paired activation then)
 __global__ __launch_bounds__(256) void dense_mv_kernel(dn_args g) {
     extern __shared__ __attribute__((aligned(16))) float xs[]; // [C][Kp]
     long long row0;
     int T;
     dn_rows(g, row0, T);
     const long long K = g.K, Kp = (K + 7) / 8 * 8;
-    for (long long i = threadIdx.x; i < (long long)C * Kp; i += 256) {
-        const int c = (int)(i / Kp);
-        const long long k = i % Kp;
-        float v = (c < T && k < K) ? dn_aval(g, row0, c, k) : 0.f;
-        if constexpr (sizeof(WT) == 2) v = dn_bf2f(dn_f2bf(v));
-        xs[i] = v;
+#pragma unroll
+    for (int c = 0; c < C; c++) {
+        const float *x = c < T ? dn_arow(g, row0, c) : nullptr, *p = g.mu && c < T ? (c ? dn_arow(g, row0, c - 1) : g.shift0) : nullptr;
+#pragma unroll 4
+        for (int k = threadIdx.x; k < (int)Kp; k += 256) {
+            float v = x && k < K ? x[k] : 0.f;
+            if (p && k < K) v += (p[k] - v) * g.mu[k]; // (the token-shift mix of dn_aval)
+            if constexpr (sizeof(WT) == 2) v = dn_bf2f(dn_f2bf(v));
+            xs[(long long)c * Kp + k] = v;
+        }
     }
     __syncthreads();
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const WT *W = (const WT *)g.w;
-    constexpr int RW = 4, VE = 16 / (int)sizeof(WT); // rows per wave at a time; elements per 16-byte load
+    constexpr int VE = 16 / (int)sizeof(WT); // elements per 16-byte load
     const bool vec = (K * (long long)sizeof(WT)) % 16 == 0;
     for (long long nb = ((long long)blockIdx.x * 4 + wave) * RW; nb < g.N; nb += (long long)gridDim.x * 4 * RW) {
         float acc[RW][C];
@@ -248,7 +253,7 @@ __global__ __launch_bounds__(256) void dense_mv_kernel(dn_args g) {
 #pragma unroll
             for (int c = 0; c < C; c++) acc[r][c] = 0.f;
         if (vec) {
-            // two 16-byte pieces of each of the four rows in flight per lane (8 KiB per wave and round)
+            // two 16-byte pieces of each row in flight per lane (four rows: 8 KiB per wave and round)
             for (long long k = (long long)lane * VE; k < K; k += 128 * VE) {
                 const long long k2 = k + 64 * VE;
                 const bool two = k2 < K;
@@ -304,7 +309,7 @@ __global__ __launch_bounds__(256) void dense_mv_kernel(dn_args g) {
 #pragma unroll
         for (int r = 0; r < RW; r++)
 #pragma unroll
-            for (int c = 0; c < C; c++) dn_put(g, c, nb + r, acc[r][c], acc[r ^ 1][c], lane == 0 && nb + r < g.N && c < T); // (nb is a multiple of four)
+            for (int c = 0; c < C; c++) dn_put(g, c, nb + r, acc[r][c], acc[RW > 1 ? (r ^ 1) : r][c], lane == 0 && nb + r < g.N && c < T); // (nb is a multiple of four)
     }
 }
 
@@ -317,12 +322,15 @@ __global__ __launch_bounds__(256) void dense_mv_grouped_kernel(dn_args g) {
     extern __shared__ __attribute__((aligned(16))) float xs[]; // [inner][Kp]
     const long long K = g.K, Kp = (K + 7) / 8 * 8;
     const int r = blockIdx.y, inner = g.g_inner;
-    for (long long i = threadIdx.x; i < (long long)inner * Kp; i += 256) {
-        const int c = (int)(i / Kp);
-        const long long k = i % Kp, s = (long long)r * inner + c;
-        float v = k < K ? g.a[(s / g.g_adiv) * g.lda + k] * (g.g_scale ? g.g_scale[s] : 1.f) : 0.f;
-        if constexpr (sizeof(WT) == 2) v = dn_bf2f(dn_f2bf(v));
-        xs[i] = v;
+    for (int c = 0; c < inner; c++) {
+        const int s = r * inner + c;
+        const float *x = g.a + (long long)(s / g.g_adiv) * g.lda, scale = g.g_scale ? g.g_scale[s] : 1.f;
+#pragma unroll 4
+        for (int k = threadIdx.x; k < (int)Kp; k += 256) {
+            float v = k < K ? x[k] * scale : 0.f;
+            if constexpr (sizeof(WT) == 2) v = dn_bf2f(dn_f2bf(v));
+            xs[(long long)c * Kp + k] = v;
+        }
     }
     __syncthreads();
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -417,8 +425,8 @@ __global__ __launch_bounds__(256) void dense_pack_kernel(dn_args g, unsigned sho
     else row0 = 0;
     const long long per_row = g.K / 8, total = (long long)Tp * per_row;
     for (long long i = (long long)blockIdx.x * 256 + threadIdx.x; i < total; i += (long long)gridDim.x * 256) {
-        const int t = (int)(i / per_row);
-        const long long k = (i % per_row) * 8;
+        const int t = (int)((unsigned)i / (unsigned)per_row); // (the packed operand has fewer than 2^31 pieces of eight)
+        const long long k = (long long)((unsigned)i % (unsigned)per_row) * 8;
         dn_us8 v;
 #pragma unroll
         for (int e = 0; e < 8; e++) v[e] = t < T ? dn_f2bf(dn_aval(g, row0, t, k + e)) : (unsigned short)0;
@@ -498,14 +506,80 @@ __global__ __launch_bounds__(256) void dense_mm_fast_kernel(dn_args g, const uns
             }
 }
 
-template <typename WT, int C>
+// Products that 128 x 128 tiles cannot spread over the chip (few outputs, or an inner size of a few steps): 32 tokens x 32 outputs per work-group.  Each of the four waves takes a
+// quarter of K, its operand fragments straight from memory (the activations are rounded to bfloat16 in registers: nothing is packed beforehand), four steps of 32 in flight; the
+// partial tiles meet in LDS.  Plain rows only (no ring, no token shift, no groups).
+__global__ __launch_bounds__(256) void dense_mm_narrow_kernel(dn_args g) {
+    __shared__ float part[4][32][33];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lq = lane >> 4, t0 = blockIdx.y * 32;
+    const long long n0 = (long long)blockIdx.x * 32, kw = g.K / 4;
+    const float *ap[2];
+    const unsigned short *bp[2];
+#pragma unroll
+    for (int i = 0; i < 2; i++) {
+        const int t = min(t0 + 16 * i + lr, g.T - 1);
+        const long long n = min(n0 + 16 * i + lr, g.N - 1);
+        ap[i] = g.a + t * g.lda + wave * kw + lq * 8;
+        bp[i] = (const unsigned short *)g.w + n * g.K + wave * kw + lq * 8;
+    }
+    dn_f4 acc[2][2];
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+#pragma unroll
+        for (int j = 0; j < 2; j++) acc[i][j] = dn_f4{0.f, 0.f, 0.f, 0.f};
+    for (long long k0 = 0; k0 < kw; k0 += 128) {
+        dn_f4 xa[4][2][2], xb[4][2];
+#pragma unroll
+        for (int u = 0; u < 4; u++) {
+            const long long k = k0 + 32 * u < kw ? k0 + 32 * u : k0; // (a step beyond the wave's share is loaded from where there is one and not used)
+#pragma unroll
+            for (int i = 0; i < 2; i++) {
+                xa[u][i][0] = *(const dn_f4 *)(ap[i] + k);
+                xa[u][i][1] = *(const dn_f4 *)(ap[i] + k + 4);
+                xb[u][i] = *(const dn_f4 *)(bp[i] + k);
+            }
+        }
+#pragma unroll
+        for (int u = 0; u < 4; u++) {
+            if (k0 + 32 * u >= kw) continue; // (uniform)
+            dn_bf8 fa[2], fb[2];
+#pragma unroll
+            for (int i = 0; i < 2; i++) {
+                dn_us8 r;
+#pragma unroll
+                for (int e = 0; e < 8; e++) r[e] = dn_f2bf(xa[u][i][e >> 2][e & 3]);
+                __builtin_memcpy(&fa[i], &r, 16);
+                __builtin_memcpy(&fb[i], &xb[u][i], 16);
+            }
+#pragma unroll
+            for (int i = 0; i < 2; i++)
+#pragma unroll
+                for (int j = 0; j < 2; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+#pragma unroll
+        for (int j = 0; j < 2; j++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) part[wave][16 * i + 4 * lq + e][16 * j + lr] = acc[i][j][e];
+    __syncthreads();
+#pragma unroll
+    for (int x = 0; x < 4; x++) {
+        const int r = (tid + 256 * x) >> 5, c = tid & 31;
+        const float v = (part[0][r][c] + part[1][r][c]) + (part[2][r][c] + part[3][r][c]);
+        dn_put(g, t0 + r, n0 + c, v, __shfl_xor(v, 1, 64), t0 + r < g.T && n0 + c < g.N); // (row n ^ 1 is the neighbouring lane's)
+    }
+}
+
+template <typename WT, int C, int RW = 4>
 static void dn_launch_mv(hipStream_t st, const dn_args &g) {
     const size_t lds = (size_t)C * ((g.K + 7) / 8 * 8) * 4;
     static unsigned long long mask = 0;
-    if (ps_first_on_device(&mask)) (void)hipFuncSetAttribute((const void *)dense_mv_kernel<WT, C>, hipFuncAttributeMaxDynamicSharedMemorySize, 64 * 1024);
-    long long blocks = (g.N + 15) / 16;
+    if (ps_first_on_device(&mask)) (void)hipFuncSetAttribute((const void *)dense_mv_kernel<WT, C, RW>, hipFuncAttributeMaxDynamicSharedMemorySize, 64 * 1024);
+    long long blocks = (g.N + 4 * RW - 1) / (4 * RW);
     if (blocks > 2048) blocks = 2048;
-    hipLaunchKernelGGL((dense_mv_kernel<WT, C>), dim3((unsigned)blocks), dim3(256), lds, st, g);
+    hipLaunchKernelGGL((dense_mv_kernel<WT, C, RW>), dim3((unsigned)blocks), dim3(256), lds, st, g);
 }
 
 int psk_dense(hipStream_t st, const psk_dense_args &a) {
@@ -556,8 +630,10 @@ int psk_dense(hipStream_t st, const psk_dense_args &a) {
     if (!a.force_tiled && a.T <= 8) {
         const int C = a.T <= 1 ? 1 : a.T <= 2 ? 2 : a.T <= 4 ? 4 : 8;
         if (kp4 * C <= 64 * 1024) {
+            const bool one_row = g.N <= 1024 && g.act != PSD_ACT_SILU_PAIR && g.act != PSD_ACT_RELU_PAIR; // (four rows per wave: at most 64 blocks)
             if (bf) {
-                if (C == 1) dn_launch_mv<unsigned short, 1>(st, g);
+                if (C == 1 && one_row) dn_launch_mv<unsigned short, 1, 1>(st, g);
+                else if (C == 1) dn_launch_mv<unsigned short, 1>(st, g);
                 else if (C == 2) dn_launch_mv<unsigned short, 2>(st, g);
                 else if (C == 4) dn_launch_mv<unsigned short, 4>(st, g);
                 else dn_launch_mv<unsigned short, 8>(st, g);
@@ -571,6 +647,11 @@ int psk_dense(hipStream_t st, const psk_dense_args &a) {
         }
     }
     const int Tp = (a.T + 127) / 128 * 128;
+    if (bf && !a.force_tiled && a.T > 8 && g.K % 128 == 0 && g.lda % 4 == 0 && ((uintptr_t)g.a & 15) == 0 && !g.mu && !g.a_mod && !g.a_step && !g.a_row0 &&
+        (g.K <= 256 || (g.N + 127) / 128 * (Tp / 128) < 32)) {
+        hipLaunchKernelGGL(dense_mm_narrow_kernel, dim3((unsigned)((g.N + 31) / 32), (unsigned)((a.T + 31) / 32)), dim3(256), 0, st, g);
+        return 0;
+    }
     if (bf && !a.force_tiled && a.T > 8 && g.K % 64 == 0 && a.pack && (size_t)Tp * g.K * 2 <= a.pack_bytes) {
         long long pb = ((long long)Tp * (g.K / 8) + 255) / 256;
         if (pb > 8192) pb = 8192;

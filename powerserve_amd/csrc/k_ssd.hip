@@ -16,6 +16,7 @@
 // finds in the state is the one its numbers are relative to.
 #include "ps_seq.h"
 
+#include <algorithm>
 #include <cmath>
 
 typedef float sd_f4 __attribute__((ext_vector_type(4)));
@@ -103,7 +104,7 @@ __global__ __launch_bounds__(1024) void mlstm_gates_kernel(const ps_seq_step *st
     }
 }
 
-// block (chunk, head); a wave takes units of 64 values x 32 state rows.  A lane's four value columns (two state rows) are neighbours: operand tile ii (jj) holds every
+// block (chunk, head, piece of the values); a wave takes units of 64 values x 32 state rows.  A lane's four value columns (two state rows) are neighbours: operand tile ii (jj) holds every
 // fourth (second) one, and a result goes back to its place at the store.
 template <bool LSTM>
 __global__ __launch_bounds__(256) void ssd_state_kernel(const float *x, const float *B, long long ld, const float *dtraw, long long ldb, const float *a_log, const float *dt_bias, int H,
@@ -122,7 +123,7 @@ __global__ __launch_bounds__(256) void ssd_state_kernel(const float *x, const fl
     const float *xh = x + (long long)h * P, *Bh = B + (long long)(h / (H / G)) * N;
     float *Uh = U + ((long long)blockIdx.x * H + h) * (P + (LSTM ? 1 : 0)) * N;
     if constexpr (LSTM) { // the column of ones
-        for (int n = tid; n < N; n += 256) {
+        for (int n = tid; blockIdx.z == 0 && n < N; n += 256) {
             float a = 0.f;
 #pragma unroll 16
             for (int s = 0; s < SD_Q; s++) a = fmaf(ws[s], Bh[(long long)(t0 + s < T ? t0 + s : T - 1) * ld + n], a);
@@ -130,7 +131,7 @@ __global__ __launch_bounds__(256) void ssd_state_kernel(const float *x, const fl
         }
     }
     const int nJ = (N + 31) / 32, units = (P + 63) / 64 * nJ;
-    for (int u = wave; u < units; u += 4) {
+    for (int u = wave + 4 * (int)blockIdx.z; u < units; u += 4 * (int)gridDim.z) {
         const int p = u / nJ * 64 + 4 * lr, n = u % nJ * 32 + 2 * lr;
         sd_f4 acc[4][2];
 #pragma unroll
@@ -386,7 +387,7 @@ void psk_mlstm_chunked(hipStream_t st, const ps_seq_step *step, int64_t state_of
     G.dec = G.tail + per;
     hipLaunchKernelGGL(mlstm_gates_kernel, dim3(H), dim3(64 * (chunks < 16 ? chunks : 16)), (size_t)chunks * 16 + (size_t)(chunks + 1) * 4, st, step, (long long)m_off, iraw, fraw,
                        (long long)ldb, cap, H, T, chunks, G, mt);
-    hipLaunchKernelGGL(ssd_state_kernel<true>, dim3(chunks, H), dim3(256), 0, st, v, k, (long long)ld, nullptr, 0ll, nullptr, nullptr, H, H, d, dv, T, U, nullptr, G);
+    hipLaunchKernelGGL(ssd_state_kernel<true>, dim3(chunks, H, (unsigned)std::max(1, ((dv + 63) / 64 * ((d + 31) / 32) + 3) / 4)), dim3(256), 0, st, v, k, (long long)ld, nullptr, 0ll, nullptr, nullptr, H, H, d, dv, T, U, nullptr, G);
     const long long per_head = (long long)(dv + 1) * d / 4;
     hipLaunchKernelGGL(ssd_pass_kernel, dim3((unsigned)((per_head * H + 255) / 256)), dim3(256), 0, st, step, (long long)state_off, U, G.dec, H, per_head, chunks);
     const size_t lds = (size_t)4 * (16 * (d + 4) + 16 * 17) * 4;
@@ -395,7 +396,9 @@ void psk_mlstm_chunked(hipStream_t st, const ps_seq_step *step, int64_t state_of
         (void)hipFuncSetAttribute((const void *)ssd_out_kernel<4, true>, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
         (void)hipFuncSetAttribute((const void *)ssd_out_kernel<8, true>, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
     }
-    const auto kernel = dv <= 64 ? ssd_out_kernel<4, true> : ssd_out_kernel<8, true>;
-    hipLaunchKernelGGL(kernel, dim3(chunks, H, dv <= 64 ? 1 : (dv + 127) / 128), dim3(256), lds, st, v, k, q, (long long)ld, nullptr, 0ll, nullptr, nullptr, nullptr, U, H, H, d, dv, T, o,
+    // pieces of 64 values where pieces of 128 would leave CUs without a block
+    const bool small = dv <= 64 || (long long)chunks * H * ((dv + 127) / 128) < 512;
+    const auto kernel = small ? ssd_out_kernel<4, true> : ssd_out_kernel<8, true>;
+    hipLaunchKernelGGL(kernel, dim3(chunks, H, small ? (dv + 63) / 64 : (dv + 127) / 128), dim3(256), lds, st, v, k, q, (long long)ld, nullptr, 0ll, nullptr, nullptr, nullptr, U, H, H, d, dv, T, o,
                        (long long)ldo, G, 1.f / sqrtf((float)d), nq);
 }
