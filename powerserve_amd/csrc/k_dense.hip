@@ -2,7 +2,7 @@
 // fp32 throughout on v_mfma_f32_16x16x4_f32 (one rounding per product, fp32 adds: a true fp32 product, no reduced-precision mode).
 //   dense_mm_kernel<WT>   tiled mat-mul, 64 tokens x 64 outputs per work-group of four waves, any T / N / K (edges zero-filled)
 //   dense_mm_fast_kernel  bf16, K % 64 == 0, more than 8 tokens: 128 x 128 tiles over an operand packed to bf16 by dense_pack_kernel
-//   dense_mm_narrow_kernel bf16, K % 128 == 0, more than 8 tokens, products too small to fill the chip with 128 x 128 tiles: 32 x 32 tiles, the four waves share K
+//   dense_mm_narrow_kernel bf16, K % 128 == 0, more than 8 tokens, products too small to fill the chip with 128 x 128 tiles: 32 x 32 tiles, the waves share K
 //   dense_mv_kernel<WT,C,RW> a few tokens (C <= 8 columns): the activation rows live in LDS, a wave streams RW weight rows at a time
 // All take the same operand description (ps_seq.h psk_dense_args): ring rows, the token-shift mix and the epilogue
 // (bias, activation, scale, a factor from a second table) are part of the launch, so no mixer needs a kernel of its own around its projections.
@@ -506,13 +506,14 @@ __global__ __launch_bounds__(256) void dense_mm_fast_kernel(dn_args g, const uns
             }
 }
 
-// Products that 128 x 128 tiles cannot spread over the chip (few outputs, or an inner size of a few steps): 32 tokens x 32 outputs per work-group.  Each of the four waves takes a
-// quarter of K, its operand fragments straight from memory (the activations are rounded to bfloat16 in registers: nothing is packed beforehand), four steps of 32 in flight; the
+// Products that 128 x 128 tiles cannot spread over the chip (few outputs, or an inner size of a few steps): 32 tokens x 32 outputs per work-group.  Each of the NW waves takes
+// its share of K, its operand fragments straight from memory (the activations are rounded to bfloat16 in registers: nothing is packed beforehand), four steps of 32 in flight; the
 // partial tiles meet in LDS.  Plain rows only (no ring, no token shift, no groups).
-__global__ __launch_bounds__(256) void dense_mm_narrow_kernel(dn_args g) {
-    __shared__ float part[4][32][33];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lq = lane >> 4, t0 = blockIdx.y * 32;
-    const long long n0 = (long long)blockIdx.x * 32, kw = g.K / 4;
+template <int NW>
+__global__ __launch_bounds__(64 * NW) void dense_mm_narrow_kernel(dn_args g) {
+    __shared__ float part[NW][32][33];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lq = lane >> 4, t0 = blockIdx.x * 32; // (rows fastest: the blocks that read the same rows of A sit on one XCD where the row tiles are a multiple of 8)
+    const long long n0 = (long long)blockIdx.y * 32, kw = g.K / NW;
     const float *ap[2];
     const unsigned short *bp[2];
 #pragma unroll
@@ -565,9 +566,11 @@ __global__ __launch_bounds__(256) void dense_mm_narrow_kernel(dn_args g) {
             for (int e = 0; e < 4; e++) part[wave][16 * i + 4 * lq + e][16 * j + lr] = acc[i][j][e];
     __syncthreads();
 #pragma unroll
-    for (int x = 0; x < 4; x++) {
-        const int r = (tid + 256 * x) >> 5, c = tid & 31;
-        const float v = (part[0][r][c] + part[1][r][c]) + (part[2][r][c] + part[3][r][c]);
+    for (int x = 0; x < 16 / NW; x++) {
+        const int r = (tid + 64 * NW * x) >> 5, c = tid & 31;
+        float v = part[0][r][c];
+#pragma unroll
+        for (int w = 1; w < NW; w++) v += part[w][r][c];
         dn_put(g, t0 + r, n0 + c, v, __shfl_xor(v, 1, 64), t0 + r < g.T && n0 + c < g.N); // (row n ^ 1 is the neighbouring lane's)
     }
 }
@@ -649,7 +652,9 @@ int psk_dense(hipStream_t st, const psk_dense_args &a) {
     const int Tp = (a.T + 127) / 128 * 128;
     if (bf && !a.force_tiled && a.T > 8 && g.K % 128 == 0 && g.lda % 4 == 0 && ((uintptr_t)g.a & 15) == 0 && !g.mu && !g.a_mod && !g.a_step && !g.a_row0 &&
         (g.K <= 256 || (g.N + 127) / 128 * (Tp / 128) < 32)) {
-        hipLaunchKernelGGL(dense_mm_narrow_kernel, dim3((unsigned)((g.N + 31) / 32), (unsigned)((a.T + 31) / 32)), dim3(256), 0, st, g);
+        const dim3 grid((unsigned)((a.T + 31) / 32), (unsigned)((g.N + 31) / 32));
+        if (g.K % 256 == 0 && g.K >= 1024) hipLaunchKernelGGL(dense_mm_narrow_kernel<8>, grid, dim3(512), 0, st, g);
+        else hipLaunchKernelGGL(dense_mm_narrow_kernel<4>, grid, dim3(256), 0, st, g);
         return 0;
     }
     if (bf && !a.force_tiled && a.T > 8 && g.K % 64 == 0 && a.pack && (size_t)Tp * g.K * 2 <= a.pack_bytes) {
